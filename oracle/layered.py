@@ -42,6 +42,11 @@ def one_plus_norm(x, w, eps):
     return rms(x, eps) * (1 + w)
 
 
+def xielu(z, p, q):
+    """quadratic above zero, exponential below, the two halves with a common slope at zero; p and q through softplus"""
+    return np.where(z > 0, softplus(p) * z * z, (0.5 + softplus(q)) * (np.expm1(np.minimum(z, 0)) - z)) + 0.5 * z
+
+
 def unit(x):
     return x / np.sqrt((x * x).sum(-1, keepdims=True) + 1e-6)
 
@@ -73,6 +78,17 @@ def rotate_pairs(x, pos, rot):
     u, v = x[..., 0:n:2], x[..., 1:n:2]
     y[..., 0:n:2] = u * c - v * s
     y[..., 1:n:2] = v * c + u * s
+    return y
+
+
+def rotate_halves(x, pos, rot):
+    """pairs (i, i + dims / 2) of the first rot.dims dimensions; x [..., dim]"""
+    n = rot["dims"] // 2
+    a = pos * float(rot["base"]) ** (-2 * np.arange(n, dtype=F) / rot["dims"])
+    y = x.copy()
+    u, v = x[..., :n], x[..., n:2 * n]
+    y[..., :n] = u * np.cos(a) - v * np.sin(a)
+    y[..., n:2 * n] = v * np.cos(a) + u * np.sin(a)
     return y
 
 
@@ -177,6 +193,85 @@ def channel_delta(h, W, pre, m, eps, st):
     return np.array(out)
 
 
+# ---- gated delta rule with one decay per head -----------------------------------------------------
+def head_delta(h, W, pre, m, eps, st):
+    H, G, dk, dv, taps = m["heads"], m["kv_heads"], m["dim"], m["vdim"], m["conv"]
+    if not st:
+        st.update(S=np.zeros((H, dk, dv)), q=np.zeros((taps - 1, G * dk)), k=np.zeros((taps - 1, G * dk)), v=np.zeros((taps - 1, H * dv)))
+    out = []
+    for row in h:
+        q, st["q"] = short_conv(W[pre + ".q"] @ row, W[pre + ".q.conv"], st["q"])
+        k, st["k"] = short_conv(W[pre + ".k"] @ row, W[pre + ".k.conv"], st["k"])
+        v, st["v"] = short_conv(W[pre + ".v"] @ row, W[pre + ".v.conv"], st["v"])
+        q, k, v = unit(q.reshape(G, dk)) * dk ** -0.5, unit(k.reshape(G, dk)), v.reshape(H, dv)
+        beta = sigmoid(W[pre + ".b"] @ row)
+        g = np.exp(-np.exp(W[pre + ".A_log"]) * softplus(W[pre + ".a"] @ row + W[pre + ".dt_bias"]))
+        o = np.zeros((H, dv))
+        for n in range(H):
+            kv = n // (H // G)
+            st["S"][n], o[n] = delta_step(st["S"][n], q[kv], k[kv], v[n], np.full(dk, g[n]), beta[n])
+        y = (rms(o, eps) * W[pre + ".norm"]).reshape(-1) * silu(W[pre + ".g"] @ row)
+        out.append(W[pre + ".o"] @ y)
+    return np.array(out)
+
+
+# ---- time mixing with a decay per key channel and a bonus for the current token --------------------
+def wkv_step(S, r, k, v, w, u):
+    """one head, one token; S [dim, dim]"""
+    o = (S + np.outer(u * k, v)).T @ r
+    return w[:, None] * S + np.outer(k, v), o
+
+
+def wkv(h, W, pre, m, eps, st):
+    H, d = m["heads"], m["dim"]
+    if not st:
+        st.update(S=np.zeros((H, d, d)), h=np.zeros(h.shape[1]))
+    out = []
+    for row in h:
+        mix = {s: row + (st["h"] - row) * W[f"{pre}.mu.{s}"] for s in "rkvgw"}
+        st["h"] = row
+        r, k, v = ((W[f"{pre}.{s}"] @ mix[s]).reshape(H, d) for s in "rkv")
+        w = np.exp(-np.exp(W[pre + ".w2"] @ np.tanh(W[pre + ".w1"] @ mix["w"]) + W[pre + ".w0"])).reshape(H, d)
+        o = np.zeros((H, d))
+        for n in range(H):
+            st["S"][n], o[n] = wkv_step(st["S"][n], r[n], k[n], v[n], w[n], W[pre + ".u"][n])
+        out.append(W[pre + ".o"] @ (rms(o, eps).reshape(-1) * W[pre + ".norm"] * silu(W[pre + ".g"] @ mix["g"])))
+    return np.array(out)
+
+
+# ---- latent attention in a sliding window ----------------------------------------------------------
+def latent_attention(h, W, pre, m, eps, st, p0):
+    H, dk, dr, dv, rank = m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"]
+    out = []
+    for t, row in enumerate(h):
+        pos = p0 + t
+        q = (W[pre + ".uq"] @ (rms(W[pre + ".dq"] @ row, eps) * W[pre + ".dq.norm"])).reshape(H, dk + dr)
+        kv = W[pre + ".dkv"] @ row
+        st.setdefault("c", []).append(rms(kv[:rank], eps) * W[pre + ".dkv.norm"])
+        st.setdefault("r", []).append(rotate_halves(kv[rank:], pos, m["rot"]))
+        first = max(0, pos - m["mask"]["size"] + 1)
+        C, R = np.array(st["c"][first:]), np.array(st["r"][first:])
+        K = (C @ W[pre + ".uk"].T).reshape(-1, H, dk)
+        V = (C @ W[pre + ".uv"].T).reshape(-1, H, dv)
+        qr = rotate_halves(q[:, dk:], pos, m["rot"])
+        o = np.zeros((H, dv))
+        for n in range(H):
+            s = (K[:, n] @ q[n, :dk] + R @ qr[n]) * m["scale"]
+            w = np.exp(s - s.max())
+            o[n] = (w / w.sum()) @ V[:, n]
+        out.append(W[pre + ".o"] @ o.reshape(-1))
+    return np.array(out)
+
+
+# ---- causal convolution in front of a sublayer -----------------------------------------------------
+def input_conv(h, w, st):
+    """h + conv(h), the last taps - 1 rows of h kept; w [width, taps]"""
+    taps = w.shape[1]
+    full = np.concatenate([st.get("in", np.zeros((taps - 1, h.shape[1]))), h], 0)
+    st["in"] = full[len(h):]
+    return h + sum(full[j:j + len(h)] * w[:, j] for j in range(taps))
+
+
 # ---- feed-forward ------------------------------------------------------------------------------
 def clamped_glu(h, W, pre, limit):
     g = np.minimum(W[pre + ".gate"] @ h, limit)
@@ -202,7 +297,7 @@ def moe(h, W, pre, m):
     return np.array(out)
 
 
-# ---- the model ---------------------------------------------------------------------------------
+# ---- the models --------------------------------------------------------------------------------
 class Sequence:
     """One sequence: its position and every layer's state."""
 
@@ -211,32 +306,58 @@ class Sequence:
         self.state = [{} for _ in model.c["layers"]]
 
 
+def parallel_layer(x, W, l, L, eps, st, p0):
+    """Timerax: x += mixer(norm(x)) + ff(norm(x)), one norm for both"""
+    h, pre = one_plus_norm(x, W[f"l{l}.norm1"], eps), f"l{l}.mix"
+    if L["type"] == "parallel":
+        y = parallel_mixer(h, W, pre, L["mixer"], eps, st, p0)
+    elif L["type"] == "channel_delta":
+        y = channel_delta(h, W, pre, L["mixer"], eps, st)
+    else:
+        raise ValueError(L["type"])
+    if L.get("mlp"):
+        y = y + moe(h, W, f"l{l}.mlp", L["mlp"])
+    return x + y
+
+
+def sandwich_layer(x, W, l, L, eps, st, p0):
+    """Ranutar: a norm before and behind each sublayer, a causal convolution over time in front of each"""
+    p, m = f"l{l}", L["mixer"]
+    h = input_conv(one_plus_norm(x, W[p + ".norm1"], eps), W[p + ".canon1"], st.setdefault("conv1", {}))
+    s = st.setdefault("mix", {})
+    if L["type"] == "wkv":
+        y = wkv(h, W, p + ".mix", m, eps, s)
+    elif L["type"] == "delta":
+        y = head_delta(h, W, p + ".mix", m, eps, s)
+    elif L["type"] == "latent_attention":
+        y = latent_attention(h, W, p + ".mix", m, eps, s, p0)
+    else:
+        raise ValueError(L["type"])
+    x = x + one_plus_norm(y, W[p + ".norm1b"], eps)
+    if L.get("mlp"):
+        h = input_conv(one_plus_norm(x, W[p + ".norm2"], eps), W[p + ".canon2"], st.setdefault("conv2", {}))
+        y = xielu(h @ W[p + ".mlp.up"].T, *W[p + ".mlp.act"]) @ W[p + ".mlp.down"].T
+        x = x + one_plus_norm(y, W[p + ".norm2b"], eps)
+    return x
+
+
 class Model:
-    """A parallel-residual model: x += mixer(norm(x)) + ff(norm(x)) per layer, one norm for both."""
+    LAYER = {"Timerax": parallel_layer, "Ranutar": sandwich_layer}
 
     def __init__(self, config, tensors):
         self.c = config
         self.W = {k: np.asarray(v, F) for k, v in tensors.items()}
+        self.layer = self.LAYER[config["architecture"]]
 
     def run(self, seq, tokens, trace=None):
         """logits [tokens, vocab]; trace: a list that gets the residual stream after every layer"""
         c, W, eps = self.c, self.W, self.c["norm"]["eps"]
         x = W["embed"][np.asarray(tokens)]
         for l, L in enumerate(c["layers"]):
-            h = one_plus_norm(x, W[f"l{l}.norm1"], eps)
-            st, pre = seq.state[l], f"l{l}.mix"
-            if L["type"] == "parallel":
-                y = parallel_mixer(h, W, pre, L["mixer"], eps, st, seq.pos)
-            elif L["type"] == "channel_delta":
-                y = channel_delta(h, W, pre, L["mixer"], eps, st)
-            else:
-                raise ValueError(L["type"])
-            if L.get("mlp"):
-                y = y + moe(h, W, f"l{l}.mlp", L["mlp"])
-            x = x + y
+            x = self.layer(x, W, l, L, eps, seq.state[l], seq.pos)
             if trace is not None:
                 trace.append(x.copy())
         seq.pos += len(tokens)
-        z = one_plus_norm(x, W["final.norm"], eps) @ W["head"].T
-        cap = c["logit_softcap"]
-        return cap * np.tanh(z / cap)
+        z = one_plus_norm(x, W["final.norm"], eps) @ W["head"].T * c.get("logit_scale", 1.0)
+        cap = c.get("logit_softcap")
+        return cap * np.tanh(z / cap) if cap else z

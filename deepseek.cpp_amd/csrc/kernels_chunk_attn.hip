@@ -2,12 +2,10 @@
 // Chunks count from position 0 of the sequence, so a sequence keeps at most one chunk of keys and values: row (position % chunk).
 //
 //   chunk_prep    rotary positions (interleaved pairs), RMS norm of q and k per head, copies of v; padded to 32 per head
-//   chunk_attn    64 queries per workgroup (16 per wave), key tiles of 32 through LDS, online softmax in 32-bit.  Scores come out of
-//                 the MFMA with the query in the lane and four keys in the registers, which is the operand order of the second
-//                 product when v's key order is permuted alike: the weights never leave their registers
+//   chunk_attn    64 queries per workgroup (attn_tile.h)
 //   chunk_store   the rows of the sequence's last chunk into its cache (behind the attention, which reads the older ones)
+#include "attn_tile.h"
 #include "layered_kernels.h"
-#include "seq_device.h"
 
 #include <math.h>
 
@@ -63,133 +61,33 @@ __global__ __launch_bounds__(256) void chunk_prep_kernel(const ChunkAttnArgs a) 
 }
 
 // ---- attention -----------------------------------------------------------------------------------------
-// LDS: a tile of 32 keys as fragments [2 x 16 keys][dim / 32][64 lanes][8], then v transposed [vdim][32 keys + pad]
+// keys and values of one head: the portion's from the workspace, older ones of the same chunk from the sequence's cache
 template <typename T>
-struct VT {
-  enum { LD = sizeof(T) == 2 ? 40 : 36 };  // elements per row of the transposed v tile
-};
-// weights x values for the 32 keys of a tile: keys 4 g + i of the first 16 and of the second 16 (g = lane / 16)
-DEV f32x4 mma_pv(const bf16* v, const f32x4& p0, const f32x4& p1, const f32x4& acc) {
-  typedef bf16 b4 __attribute__((ext_vector_type(4)));
-  const b4 v0 = *reinterpret_cast<const b4*>(v), v1 = *reinterpret_cast<const b4*>(v + 16);
-  const bf16x8 vv = __builtin_shufflevector(v0, v1, 0, 1, 2, 3, 4, 5, 6, 7);
-  const bf16x8 pp = __builtin_shufflevector(to_four<bf16>(p0), to_four<bf16>(p1), 0, 1, 2, 3, 4, 5, 6, 7);
-  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(vv, pp, acc, 0, 0, 0);
-}
-DEV f32x4 mma_pv(const float* v, const f32x4& p0, const f32x4& p1, f32x4 acc) {
-  const f32x4 v0 = *reinterpret_cast<const f32x4*>(v), v1 = *reinterpret_cast<const f32x4*>(v + 16);
-#pragma unroll
-  for (int i = 0; i < 4; ++i) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(v0[i], p0[i], acc, 0, 0, 0);
-#pragma unroll
-  for (int i = 0; i < 4; ++i) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(v1[i], p1[i], acc, 0, 0, 0);
-  return acc;
-}
-template <typename T, int KT, int VTL>  // dim_p <= 32 KT, vdim_p <= 16 VTL
-__global__ __launch_bounds__(256) void chunk_attn_kernel(const ChunkAttnArgs a) {
+struct ChunkKeys {
   typedef typename Frag<T>::type frag;
-  extern __shared__ __attribute__((aligned(16))) char lds[];
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const int h = blockIdx.y, g = h / (a.heads / a.kv_heads);
-  const SeqDesc sq = a.p.seqs[a.p.qtile[2 * blockIdx.x]];
-  const int q0 = a.p.qtile[2 * blockIdx.x + 1];          // first row of the tile inside the portion
-  const int nq = min(64, sq.len - q0);
-  const int kts = a.dim_p >> 5, vts = a.vdim_p >> 4;
-  T* kf = reinterpret_cast<T*>(lds);                     // fragments of the key tile
-  T* vt = kf + (size_t)2 * kts * 512;                    // transposed values
-  const int my_q = min(q0 + wave * 16 + (lane & 15), sq.len - 1);
-  const int my_pos = sq.pos0 + my_q, my_first = my_pos / a.chunk * a.chunk;
-  frag q[KT];
-#pragma unroll
-  for (int kt = 0; kt < KT; ++kt)
-    if (kt < kts) q[kt] = *reinterpret_cast<const frag*>(reinterpret_cast<const T*>(a.q_t) + ((size_t)(sq.row0 + my_q) * a.heads + h) * a.dim_p + kt * 32 + (lane >> 4) * 8);
-  f32x4 o[VTL];
-#pragma unroll
-  for (int i = 0; i < VTL; ++i) o[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-  float m = -INFINITY, l = 0.f;
-  const int first = (sq.pos0 + q0) / a.chunk * a.chunk, last = sq.pos0 + q0 + nq - 1;
-  const T* ck = reinterpret_cast<const T*>(sq.state + a.off_k);
-  const T* cv = reinterpret_cast<const T*>(sq.state + a.off_v);
-  auto k_row = [&](int pos) {
-    return pos >= sq.pos0 ? reinterpret_cast<const T*>(a.k_t) + ((size_t)(sq.row0 + pos - sq.pos0) * a.kv_heads + g) * a.dim_p
-                          : ck + ((size_t)(pos % a.chunk) * a.kv_heads + g) * a.dim_p;
-  };
-  auto v_row = [&](int pos) {
-    return pos >= sq.pos0 ? reinterpret_cast<const T*>(a.v_t) + ((size_t)(sq.row0 + pos - sq.pos0) * a.kv_heads + g) * a.vdim_p
-                          : cv + ((size_t)(pos % a.chunk) * a.kv_heads + g) * a.vdim_p;
-  };
-  for (int j0 = first; j0 <= last; j0 += 32) {
-    __syncthreads();
-    // keys: element groups of 8, thread -> (key, group); keys past the tile's last position repeat it (masked below)
-    const int ng = a.dim_p >> 3;
-    for (int i = tid; i < 32 * ng; i += 256) {
-      const int key = i / ng, gr = i % ng;
-      const frag f = *reinterpret_cast<const frag*>(k_row(min(j0 + key, last)) + gr * 8);
-      *reinterpret_cast<frag*>(kf + (((size_t)(key >> 4) * kts + (gr >> 2)) * 64 + (gr & 3) * 16 + (key & 15)) * 8) = f;
-    }
-    // values, transposed: thread -> (4 keys, 4 value channels)
-    const int nv = a.vdim_p >> 2;
-    for (int i = tid; i < 8 * nv; i += 256) {
-      typedef typename Frag<T>::four four;
-      const int kq = i / nv, c = (i % nv) * 4;
-      four r[4];
-#pragma unroll
-      for (int k = 0; k < 4; ++k) r[k] = *reinterpret_cast<const four*>(v_row(min(j0 + kq * 4 + k, last)) + c);
-#pragma unroll
-      for (int e = 0; e < 4; ++e) *reinterpret_cast<four*>(vt + (size_t)(c + e) * VT<T>::LD + kq * 4) = four{r[0][e], r[1][e], r[2][e], r[3][e]};
-    }
-    __syncthreads();
-    if (wave * 16 >= nq || j0 > sq.pos0 + q0 + min(wave * 16 + 15, nq - 1)) continue;  // (barriers above: every wave passes them)
-    f32x4 s[2];
-#pragma unroll
-    for (int t = 0; t < 2; ++t) {
-      s[t] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int kt = 0; kt < KT; ++kt)
-        if (kt < kts) s[t] = mma(*reinterpret_cast<const frag*>(kf + (((size_t)t * kts + kt) * 64 + lane) * 8), q[kt], s[t]);
-    }
-    float mx = m;
-#pragma unroll
-    for (int t = 0; t < 2; ++t)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int pos = j0 + t * 16 + (lane >> 4) * 4 + i;
-        s[t][i] = pos <= my_pos && pos >= my_first ? s[t][i] * a.scale : -INFINITY;
-        mx = fmaxf(mx, s[t][i]);
-      }
-    mx = fmaxf(mx, __shfl_xor(mx, 16));
-    mx = fmaxf(mx, __shfl_xor(mx, 32));
-    const float ref = mx == -INFINITY ? 0.f : mx;  // nothing visible yet: every weight below is exp(-inf) = 0
-    const float old = expf(m - ref);
-    float sum = 0.f;
-#pragma unroll
-    for (int t = 0; t < 2; ++t)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        s[t][i] = expf(s[t][i] - ref);
-        sum += s[t][i];
-      }
-    sum += __shfl_xor(sum, 16);
-    sum += __shfl_xor(sum, 32);
-    l = l * old + sum;
-    m = mx;
-#pragma unroll
-    for (int i = 0; i < VTL; ++i)
-      if (i < vts) {
-        o[i] *= old;
-        o[i] = mma_pv(vt + (size_t)(i * 16 + (lane & 15)) * VT<T>::LD + (lane >> 4) * 4, s[0], s[1], o[i]);
-      }
+  typedef typename Frag<T>::four four;
+  const ChunkAttnArgs& a;
+  const SeqDesc& s;
+  int h, g;
+  DEV int first(int pos) const { return pos / a.chunk * a.chunk; }
+  DEV frag q(int row, int gr) const { return *reinterpret_cast<const frag*>(reinterpret_cast<const T*>(a.q_t) + ((size_t)(s.row0 + row) * a.heads + h) * a.dim_p + gr * 8); }
+  DEV frag k(int pos, int gr) const {
+    const T* p = pos >= s.pos0 ? reinterpret_cast<const T*>(a.k_t) + ((size_t)(s.row0 + pos - s.pos0) * a.kv_heads + g) * a.dim_p
+                               : reinterpret_cast<const T*>(s.state + a.off_k) + ((size_t)(pos % a.chunk) * a.kv_heads + g) * a.dim_p;
+    return *reinterpret_cast<const frag*>(p + gr * 8);
   }
-  const int qi = wave * 16 + (lane & 15);
-  if (qi >= nq) return;
-  T* out = reinterpret_cast<T*>(a.out_t) + (size_t)(sq.row0 + q0 + qi) * a.out_ld + h * a.vdim;
-#pragma unroll
-  for (int i = 0; i < VTL; ++i)
-    if (i < vts)
-#pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const int c = i * 16 + (lane >> 4) * 4 + e;
-        if (c < a.vdim) out[c] = (T)(o[i][e] / l);
-      }
+  DEV four v(int pos, int c) const {
+    const T* p = pos >= s.pos0 ? reinterpret_cast<const T*>(a.v_t) + ((size_t)(s.row0 + pos - s.pos0) * a.kv_heads + g) * a.vdim_p
+                               : reinterpret_cast<const T*>(s.state + a.off_v) + ((size_t)(pos % a.chunk) * a.kv_heads + g) * a.vdim_p;
+    return *reinterpret_cast<const four*>(p + c);
+  }
+};
+template <typename T, int KT, int VTL>
+__global__ __launch_bounds__(256) void chunk_attn_kernel(const ChunkAttnArgs a) {
+  const int h = blockIdx.y;
+  const SeqDesc s = a.p.seqs[a.p.qtile[2 * blockIdx.x]];
+  attn_tile<T, KT, VTL>(ChunkKeys<T>{a, s, h, h / (a.heads / a.kv_heads)}, s, a.p.qtile[2 * blockIdx.x + 1], a.dim_p >> 5, a.vdim_p >> 4, a.vdim, a.scale,
+                        reinterpret_cast<T*>(a.out_t) + h * a.vdim, a.out_ld);
 }
 
 // ---- cache rows ------------------------------------------------------------------------------------------
@@ -218,7 +116,7 @@ int launch_chunk_prep(hipStream_t st, const ChunkAttnArgs& a, bool f32) {
 }
 template <typename T, int KT, int VTL>
 static int attn_t(hipStream_t st, const ChunkAttnArgs& a) {
-  const size_t lds = ((size_t)32 * a.dim_p + (size_t)a.vdim_p * VT<T>::LD) * sizeof(T);
+  const size_t lds = attn_tile_lds<T>(a.dim_p, a.vdim_p);
   auto k = chunk_attn_kernel<T, KT, VTL>;
   HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
   hipLaunchKernelGGL(k, dim3(a.p.n_qtiles, a.heads), dim3(256), lds, st, a);

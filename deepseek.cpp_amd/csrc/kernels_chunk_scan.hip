@@ -7,6 +7,8 @@
 //                S  <- G_16 S0 + sum_s (k_s G_16 / G_s) u_s^T
 //   mLSTM        the same without A (u = v); the decay is one number per token, exp(f + m_before - m), and k_s carries exp(i_s - m_s).
 //                A column of ones behind v makes the normaliser n one more column of S.
+//   wkv          the same without A, read before the write: o_t = (q_t G_(t-1))^T S0 + sum_{s<=t} B_ts v_s with B_ts = sum_d q_t k_s
+//                G_(t-1) / G_s below the diagonal, and the bonus on it: B_tt = sum_d q_t u k_t
 // *_prepare: everything that does not depend on S0, for all chunks at once - the operands with decays multiplied in, B, and
 // T = (I + diag(beta) A)^-1 diag(beta), so that U = T (V - Kg S0).  chunk_scan: one workgroup per (16 columns, head, sequence)
 // goes through the chunks; its 4 waves share the key channels.  S stays in MFMA accumulators: their layout (column = lane % 16, rows
@@ -48,7 +50,7 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(const DeltaArgs a, f
     const bool in = t < n && d < dim;
     sk[i] = in ? a.k[(row0 + t) * nq + (size_t)kv * dim + d] : 0.f;
     sq[i] = in ? a.q[(row0 + t) * nq + (size_t)kv * dim + d] : 0.f;
-    sg[i] = in ? a.g[(row0 + t) * a.heads * dim + (size_t)h * dim + d] : 1.f;
+    sg[i] = in ? (a.head_decay ? a.g[(row0 + t) * a.heads + h] : a.g[(row0 + t) * a.heads * dim + (size_t)h * dim + d]) : 1.f;
   }
   if (tid < 16) sb[tid] = tid < n ? a.beta[(row0 + tid) * a.heads + h] : 0.f;
   __syncthreads();
@@ -199,6 +201,65 @@ __global__ __launch_bounds__(256) void mlstm_prepare_kernel(const MlstmArgs a, c
   }
 }
 
+// ---- wkv: operands ------------------------------------------------------------------------------------------------
+template <typename T>
+__global__ __launch_bounds__(256) void wkv_prepare_kernel(const WkvArgs a, float* __restrict__ base) {
+  extern __shared__ float lds[];
+  const int tid = threadIdx.x, h = blockIdx.y, dim = a.dim, dp = (dim + 15) / 16 * 16;
+  float *sk = lds, *sq = sk + 16 * dp, *sg = sq + 16 * dp, *su = sg + 16 * dp;
+  const SeqDesc s = a.p.seqs[a.p.chunk[2 * blockIdx.x]];
+  const int t0 = a.p.chunk[2 * blockIdx.x + 1], n = min((int)CH, s.len - t0);
+  const size_t row0 = (size_t)s.row0 + t0;
+  for (int i = tid; i < 16 * dp; i += 256) {  // rows past the end: no key, no query, no decay
+    const int t = i / dp, d = i % dp;
+    const bool in = t < n && d < dim;
+    const size_t row = row0 + (in ? t : 0);
+    const int c = h * dim + (in ? d : 0);
+    const T* P = reinterpret_cast<const T*>(a.proj_t) + row * a.ld + c;
+    sk[i] = in ? (float)P[a.col_k] : 0.f;
+    sq[i] = in ? (float)P[a.col_r] : 0.f;
+    sg[i] = in ? expf(-expf(a.low_f[row * a.ld_low + c] + a.w0[c])) : 1.f;
+  }
+  for (int d = tid; d < dp; d += 256) su[d] = d < dim ? a.u[h * dim + d] : 0.f;
+  __syncthreads();
+  const Ops o = ops_at(base, blockIdx.x, a.heads, h, dim);
+  for (int d = tid; d < dp; d += 256) {
+    float G = 1.f;
+#pragma unroll
+    for (int t = 0; t < 16; ++t) {
+      o.qg[t * dp + d] = sq[t * dp + d] * G;
+      G *= sg[t * dp + d];
+    }
+    o.gend[d] = G;
+    float E = 1.f, e[16];
+#pragma unroll
+    for (int t = 15; t >= 0; --t) {
+      e[t] = sk[t * dp + d] * E;
+      E *= sg[t * dp + d];
+    }
+#pragma unroll
+    for (int t = 0; t < 16; t += 4) *reinterpret_cast<f32x4*>(o.ke + (size_t)d * 16 + t) = f32x4{e[t], e[t + 1], e[t + 2], e[t + 3]};
+  }
+  const int sx = tid >> 4, dg = tid & 15;
+  float acc[16];
+#pragma unroll
+  for (int t = 0; t < 16; ++t) acc[t] = 0.f;
+  for (int d = dg; d < dp; d += 16) {
+    float w = 0.f;
+    const float ks = sk[sx * dp + d];
+#pragma unroll
+    for (int t = 0; t < 16; ++t) {
+      acc[t] += sq[t * dp + d] * (t == sx ? ks * su[d] : w);
+      w = t == sx ? ks : w * sg[t * dp + d];
+    }
+  }
+#pragma unroll
+  for (int t = 0; t < 16; ++t) {
+    const float B = row_sum(acc[t]);
+    if (dg == t) o.b[t * 16 + sx] = sx <= t ? B : 0.f;
+  }
+}
+
 // ---- the chunks of a sequence, one after the other -------------------------------------------------------------
 struct ScanArgs {
   PassDesc p;
@@ -209,17 +270,19 @@ struct ScanArgs {
   float* o;            // [rows][heads][cols]
   size_t off_s, off_n;
 };
-template <typename T, bool DELTA, int NTL>
+enum { SCAN_DELTA, SCAN_MLSTM, SCAN_WKV };
+template <typename T, int KIND, int NTL>
 __global__ __launch_bounds__(256) void chunk_scan_kernel(const ScanArgs a) {
+  constexpr bool DELTA = KIND == SCAN_DELTA, NORM = KIND == SCAN_MLSTM;
   __shared__ __attribute__((aligned(16))) f32x4 ex[2][4][2][64];
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), g = lane >> 4, c16 = lane & 15;
   const int h = blockIdx.y, dp = (a.dim + 15) / 16 * 16, tiles = dp >> 4;
-  const int cols = DELTA ? a.vdim : a.vdim + 1;
+  const int cols = NORM ? a.vdim + 1 : a.vdim;
   const int col = blockIdx.x * 16 + c16;
-  const bool live = col < cols, norm = !DELTA && col == a.vdim;
+  const bool live = col < cols, norm = NORM && col == a.vdim;
   const SeqDesc s = a.p.seqs[blockIdx.z];
   float* S0 = reinterpret_cast<float*>(s.state + a.off_s) + (size_t)h * a.dim * a.vdim;
-  float* N0 = DELTA ? nullptr : reinterpret_cast<float*>(s.state + a.off_n) + (size_t)h * a.dim;
+  float* N0 = !NORM ? nullptr : reinterpret_cast<float*>(s.state + a.off_n) + (size_t)h * a.dim;
   const size_t nn = (size_t)a.heads * a.dim;
   f32x4 S[NTL];
 #pragma unroll
@@ -318,13 +381,13 @@ __global__ __launch_bounds__(256) void chunk_scan_kernel(const ScanArgs a) {
 }
 
 // ---- launches ------------------------------------------------------------------------------------------------------
-template <typename T, bool DELTA>
+template <typename T, int KIND>
 static int scan_t(hipStream_t st, const ScanArgs& a) {
   if (a.dim < 1 || a.dim > RECUR_MAX_DIM) DSK_FAIL(DSK_ERR_UNSUPPORTED, "recurrence: key size %d (max %d)", a.dim, (int)RECUR_MAX_DIM);
-  const dim3 grid(cdiv(DELTA ? a.vdim : a.vdim + 1, 16), a.heads, a.p.n_seqs);
-  if (a.dim <= 64) hipLaunchKernelGGL((chunk_scan_kernel<T, DELTA, 1>), grid, dim3(256), 0, st, a);
-  else if (a.dim <= 128) hipLaunchKernelGGL((chunk_scan_kernel<T, DELTA, 2>), grid, dim3(256), 0, st, a);
-  else hipLaunchKernelGGL((chunk_scan_kernel<T, DELTA, 4>), grid, dim3(256), 0, st, a);
+  const dim3 grid(cdiv(KIND == SCAN_MLSTM ? a.vdim + 1 : a.vdim, 16), a.heads, a.p.n_seqs);
+  if (a.dim <= 64) hipLaunchKernelGGL((chunk_scan_kernel<T, KIND, 1>), grid, dim3(256), 0, st, a);
+  else if (a.dim <= 128) hipLaunchKernelGGL((chunk_scan_kernel<T, KIND, 2>), grid, dim3(256), 0, st, a);
+  else hipLaunchKernelGGL((chunk_scan_kernel<T, KIND, 4>), grid, dim3(256), 0, st, a);
   return DSK_OK;
 }
 int launch_delta_chunks(hipStream_t st, const DeltaArgs& a, const ChunkScan& c) {
@@ -332,13 +395,21 @@ int launch_delta_chunks(hipStream_t st, const DeltaArgs& a, const ChunkScan& c) 
   const size_t lds = ((size_t)48 * dp + 16 * 17 + 16) * 4;
   HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void*>(delta_prepare_kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
   hipLaunchKernelGGL(delta_prepare_kernel, dim3(a.p.n_chunks, a.heads), dim3(256), lds, st, a, c.ops);
-  return scan_t<float, true>(st, ScanArgs{a.p, a.heads, a.dim, a.vdim, c.ops, a.v, a.heads * a.vdim, a.o, a.off_s, 0});
+  return scan_t<float, SCAN_DELTA>(st, ScanArgs{a.p, a.heads, a.dim, a.vdim, c.ops, a.v, a.heads * a.vdim, a.o, a.off_s, 0});
 }
 template <typename T>
 static int mlstm_t(hipStream_t st, const MlstmArgs& a, const ChunkScan& c) {
   const int dp = (a.dim + 15) / 16 * 16;
   hipLaunchKernelGGL(mlstm_gates_kernel, dim3(a.heads, a.p.n_seqs), dim3(64), 0, st, a, c);
   hipLaunchKernelGGL(mlstm_prepare_kernel<T>, dim3(a.p.n_chunks, a.heads), dim3(256), ((size_t)32 * dp + 32) * 4, st, a, c);
-  return scan_t<T, false>(st, ScanArgs{a.p, a.heads, a.dim, a.vdim, c.ops, reinterpret_cast<const T*>(a.proj_t) + a.col_v, a.ld, a.o, a.off_s, a.off_n});
+  return scan_t<T, SCAN_MLSTM>(st, ScanArgs{a.p, a.heads, a.dim, a.vdim, c.ops, reinterpret_cast<const T*>(a.proj_t) + a.col_v, a.ld, a.o, a.off_s, a.off_n});
 }
 int launch_mlstm_chunks(hipStream_t st, const MlstmArgs& a, const ChunkScan& c, bool f32) { return f32 ? mlstm_t<float>(st, a, c) : mlstm_t<bf16>(st, a, c); }
+template <typename T>
+static int wkv_t(hipStream_t st, const WkvArgs& a, const ChunkScan& c) {
+  if (a.dim > RECUR_MAX_DIM) DSK_FAIL(DSK_ERR_UNSUPPORTED, "wkv: key size %d (max %d)", a.dim, (int)RECUR_MAX_DIM);
+  const int dp = (a.dim + 15) / 16 * 16;
+  hipLaunchKernelGGL(wkv_prepare_kernel<T>, dim3(a.p.n_chunks, a.heads), dim3(256), (size_t)49 * dp * 4, st, a, c.ops);
+  return scan_t<T, SCAN_WKV>(st, ScanArgs{a.p, a.heads, a.dim, a.dim, c.ops, reinterpret_cast<const T*>(a.proj_t) + a.col_v, a.ld, a.o, a.off_s, 0});
+}
+int launch_wkv_chunks(hipStream_t st, const WkvArgs& a, const ChunkScan& c, bool f32) { return f32 ? wkv_t<float>(st, a, c) : wkv_t<bf16>(st, a, c); }

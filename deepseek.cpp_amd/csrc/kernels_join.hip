@@ -1,5 +1,5 @@
-// kernels_join.hip -- between the matrix products of layered models: the 32-bit residual sum with the norm behind it, and the
-// router's choice of experts.
+// kernels_join.hip -- between the matrix products of layered models: the 32-bit residual sum with the norm behind it, the causal
+// convolution and the blends with the previous token that may follow the norm, and the router's choice of experts.
 #include "layered_kernels.h"
 #include "route_device.h"
 #include "seq_device.h"
@@ -27,6 +27,51 @@ DEV void store_v(S* p, const float (&v)[V]) {
   } else {
     p[0] = (S)v[0];
   }
+}
+// y, or its blends with the previous token's y, of V channels from c on
+template <typename T, int V>
+DEV void store_blends(const ConvArgs& a, int D, int row, int c, const float (&y)[V], const float (&prev)[V]) {
+  T* out = reinterpret_cast<T*>(a.out_t) + (size_t)row * a.ld + c;
+  if (!a.mu) {
+    store_v<T, V>(out, y);
+    return;
+  }
+  for (int s = 0; s < a.n_mix; ++s) {
+    float m[V];
+    load_v<float, V>(a.mu + (size_t)s * D + c, true, m);
+#pragma unroll
+    for (int e = 0; e < V; ++e) m[e] = y[e] + (prev[e] - y[e]) * m[e];
+    store_v<T, V>(out + s * a.mix_stride, m);
+  }
+}
+// a sequence's only token of the pass: V channels of h through the convolution; keeps the inputs (and y) for the next token
+template <typename T, int V>
+DEV void conv_one(const JoinArgs& j, int row, int c, const float (&h)[V]) {
+  const ConvArgs& a = j.conv;
+  const SeqDesc s = j.p.seqs[j.p.row_seq[row]];
+  const int D = j.width, taps = a.taps;
+  const float* hist = reinterpret_cast<const float*>(s.state + a.off_in) + (size_t)s.flip * (taps - 1) * D + c;
+  float* next = reinterpret_cast<float*>(s.state + a.off_in) + (size_t)(s.flip ^ 1) * (taps - 1) * D + c;
+  float y[V], prev[V];
+#pragma unroll
+  for (int e = 0; e < V; ++e) y[e] = 0.f;
+#pragma unroll 4
+  for (int t = 0; t < taps - 1; ++t) {
+    float old[V];
+    load_v<float, V>(hist + (size_t)t * D, s.pos0 - (taps - 1) + t >= 0, old);
+#pragma unroll
+    for (int e = 0; e < V; ++e) y[e] += old[e] * a.w[(size_t)(c + e) * taps + t];
+    if (t > 0) store_v<float, V>(next + (size_t)(t - 1) * D, old);
+  }
+  if (taps > 1) store_v<float, V>(next + (size_t)(taps - 2) * D, h);
+#pragma unroll
+  for (int e = 0; e < V; ++e) y[e] = h[e] + (y[e] + h[e] * a.w[(size_t)(c + e) * taps + taps - 1]);
+  if (a.mu) {
+    float* P = reinterpret_cast<float*>(s.state + a.off_prev) + c;
+    load_v<float, V>(P + (size_t)s.flip * D, s.pos0 > 0, prev);
+    store_v<float, V>(P + (size_t)(s.flip ^ 1) * D, y);
+  }
+  store_blends<T, V>(a, D, row, c, y, prev);
 }
 template <typename T, int NT, int VPT, int V>
 __global__ __launch_bounds__(NT) void join_kernel(const JoinArgs a) {
@@ -75,6 +120,21 @@ __global__ __launch_bounds__(NT) void join_kernel(const JoinArgs a) {
 #pragma unroll
         for (int e = 0; e < V; ++e) add[i][e] = 0.5f * (add[i][e] * ra * wa[e] + vb[i][e] * rb * wb[e]);
       }
+    } else if (a.post_w) {
+      float sa = 0.f;
+#pragma unroll
+      for (int i = 0; i < VPT; ++i)
+#pragma unroll
+        for (int e = 0; e < V; ++e) sa += add[i][e] * add[i][e];
+      sa = block_sum<NT>(sa, red);
+      const float ra = 1.f / sqrtf(sa / D + a.eps);
+#pragma unroll
+      for (int i = 0; i < VPT; ++i) {
+        float w[V];
+        load_v<float, V>(a.post_w + at(i), at(i) < D, w);
+#pragma unroll
+        for (int e = 0; e < V; ++e) add[i][e] *= ra * (w[e] + a.norm_offset);
+      }
     }
   }
   if (a.y_t) {
@@ -113,7 +173,9 @@ __global__ __launch_bounds__(NT) void join_kernel(const JoinArgs a) {
     load_v<float, V>(a.norm_w + at(i), true, w);
 #pragma unroll
     for (int e = 0; e < V; ++e) w[e] = x[i][e] * r * (w[e] + a.norm_offset);
-    store_v<T, V>(h + at(i), w);
+    if (a.conv.w) conv_one<T, V>(a, row, at(i), w);
+    else if (a.h_f) store_v<float, V>(a.h_f + (size_t)row * D + at(i), w);
+    else store_v<T, V>(h + at(i), w);
   }
 }
 template <typename T>
@@ -137,6 +199,113 @@ int launch_join(hipStream_t st, const JoinArgs& a, bool f32) {
   const int n = a.only_want ? a.p.n_want : a.p.rows;
   if (n < 1) DSK_FAIL(DSK_ERR_INVALID, "join: no rows");
   return f32 ? join_t<float>(st, a, n) : join_t<bf16>(st, a, n);
+}
+
+// ---- convolution in front of a sublayer, portions --------------------------------------------------------
+// A thread takes V channels of the (up to 16) rows of a chunk; TAPS = 0: any number of taps, read from memory again and again.
+template <typename T, int V, int TAPS>
+__global__ __launch_bounds__(256) void conv_kernel(const PassDesc p, int D, const float* __restrict__ h_f, const ConvArgs a) {
+  constexpr int R = RECUR_CHUNK, K = TAPS ? TAPS : 1;
+  const int c = V * (blockIdx.y * 256 + threadIdx.x), taps = TAPS ? TAPS : a.taps;
+  if (c >= D) return;
+  const SeqDesc s = p.seqs[p.chunk[2 * blockIdx.x]];
+  const int t0 = p.chunk[2 * blockIdx.x + 1], n_rows = min(R, s.len - t0);
+  const float* H = h_f + (size_t)s.row0 * D + c;
+  const float* hist = reinterpret_cast<const float*>(s.state + a.off_in) + (size_t)s.flip * (taps - 1) * D + c;
+  float* P = a.mu ? reinterpret_cast<float*>(s.state + a.off_prev) + c : nullptr;
+  auto input = [&](int u, float (&v)[V]) {  // row u of the portion; before it: the kept inputs, zero before the sequence's start
+    if (u >= 0) load_v<float, V>(H + (size_t)u * D, true, v);
+    else load_v<float, V>(hist + (size_t)(max(u, 1 - taps) + taps - 1) * D, u >= 1 - taps && s.pos0 + u >= 0, v);
+  };
+  float y[V], prev[V];
+  const bool has_prev = a.mu != nullptr;
+  if constexpr (TAPS > 1) {
+    float w[V][K], x[R + K][V];  // inputs t0 - taps .. t0 + 15 (the first one only for the previous token's y)
+#pragma unroll
+    for (int e = 0; e < V; ++e)
+#pragma unroll
+      for (int j = 0; j < K; ++j) w[e][j] = a.w[(size_t)(c + e) * K + j];
+#pragma unroll
+    for (int r = 0; r < R + K; ++r) input(min(t0 - K + r, s.len - 1), x[r]);
+    auto conv = [&](int t, float (&out)[V]) {  // of input x[t + K]
+#pragma unroll
+      for (int e = 0; e < V; ++e) {
+        float z = 0.f;
+#pragma unroll
+        for (int j = 0; j < K; ++j) z += x[t + 1 + j][e] * w[e][j];
+        out[e] = x[t + K][e] + z;
+      }
+    };
+    float ys[R + 1][V];  // behind the previous token's
+    if (has_prev && t0 == 0) load_v<float, V>(P + (size_t)s.flip * D, s.pos0 > 0, ys[0]);
+    else conv(-1, ys[0]);
+#pragma unroll
+    for (int t = 0; t < R; ++t) conv(t, ys[t + 1]);
+    T* out = reinterpret_cast<T*>(a.out_t) + (size_t)(s.row0 + t0) * a.ld + c;
+    for (int i = 0; i < (has_prev ? a.n_mix : 1); ++i) {
+      float mu[V];
+      load_v<float, V>(has_prev ? a.mu + (size_t)i * D + c : a.w, has_prev, mu);
+#pragma unroll
+      for (int t = 0; t < R; ++t) {
+        float v[V];
+#pragma unroll
+        for (int e = 0; e < V; ++e) v[e] = ys[t + 1][e] + (ys[t][e] - ys[t + 1][e]) * mu[e];
+        if (t < n_rows) store_v<T, V>(out + i * a.mix_stride + (size_t)t * a.ld, v);
+      }
+    }
+#pragma unroll
+    for (int t = 0; t < R; ++t)
+#pragma unroll
+      for (int e = 0; e < V; ++e)
+        if (t < n_rows) y[e] = ys[t + 1][e];
+  } else {
+    auto conv = [&](int u, float (&out)[V]) {
+      float x[V];
+#pragma unroll
+      for (int e = 0; e < V; ++e) out[e] = 0.f;
+      for (int j = 0; j < taps; ++j) {
+        input(u - (taps - 1) + j, x);
+#pragma unroll
+        for (int e = 0; e < V; ++e) out[e] += x[e] * a.w[(size_t)(c + e) * taps + j];
+      }
+#pragma unroll
+      for (int e = 0; e < V; ++e) out[e] += x[e];
+    };
+    if (has_prev) {
+      if (t0 == 0) load_v<float, V>(P + (size_t)s.flip * D, s.pos0 > 0, prev);
+      else conv(t0 - 1, prev);
+    }
+    for (int t = 0; t < n_rows; ++t) {
+      conv(t0 + t, y);
+      store_blends<T, V>(a, D, s.row0 + t0 + t, c, y, prev);
+#pragma unroll
+      for (int e = 0; e < V; ++e) prev[e] = y[e];
+    }
+  }
+  if (t0 + n_rows < s.len) return;
+  float* next = reinterpret_cast<float*>(s.state + a.off_in) + (size_t)(s.flip ^ 1) * (taps - 1) * D + c;
+  for (int j = 0; j < taps - 1; ++j) {  // the portion's end: what the next one needs, in the other copy
+    float x[V];
+    input(s.len - (taps - 1) + j, x);
+    store_v<float, V>(next + (size_t)j * D, x);
+  }
+  if (has_prev) store_v<float, V>(P + (size_t)(s.flip ^ 1) * D, y);
+}
+template <typename T, int V>
+static void conv_t(hipStream_t st, const PassDesc& p, int D, const float* h_f, const ConvArgs& a) {
+  const dim3 grid(p.n_chunks, (D / V + 255) / 256);
+  switch (a.taps) {
+    case 2: hipLaunchKernelGGL((conv_kernel<T, V, 2>), grid, dim3(256), 0, st, p, D, h_f, a); break;
+    case 3: hipLaunchKernelGGL((conv_kernel<T, V, 3>), grid, dim3(256), 0, st, p, D, h_f, a); break;
+    case 4: hipLaunchKernelGGL((conv_kernel<T, V, 4>), grid, dim3(256), 0, st, p, D, h_f, a); break;
+    default: hipLaunchKernelGGL((conv_kernel<T, V, 0>), grid, dim3(256), 0, st, p, D, h_f, a);
+  }
+}
+int launch_conv(hipStream_t st, const PassDesc& p, int width, const float* h_f, const ConvArgs& a, bool f32) {
+  if (a.taps < 1 || width < 1 || p.n_chunks < 1) DSK_FAIL(DSK_ERR_INVALID, "conv: width %d, %d taps", width, a.taps);
+  if (width & 3) f32 ? conv_t<float, 1>(st, p, width, h_f, a) : conv_t<bf16, 1>(st, p, width, h_f, a);
+  else f32 ? conv_t<float, 4>(st, p, width, h_f, a) : conv_t<bf16, 4>(st, p, width, h_f, a);
+  return DSK_OK;
 }
 
 // ---- router ----------------------------------------------------------------------------------------

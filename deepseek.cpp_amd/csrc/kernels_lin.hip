@@ -17,18 +17,18 @@ static int cdiv(int a, int b) { return (a + b - 1) / b; }
 
 // ---- packing -----------------------------------------------------------------------------------
 __global__ __launch_bounds__(256) void pack_kernel(const uint16_t* __restrict__ src, int rows, int k, uint16_t* __restrict__ dst, int kt, int row0, int col0,
-                                                   int interleave) {
+                                                   int interleave, int transpose) {
   const size_t n = (size_t)rows * k;
   for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (size_t)gridDim.x * 256) {
-    const int r = (int)(i / k), c = (int)(i % k) + col0;
+    const int r = (int)(transpose ? i % k : i / k), c = (int)(transpose ? i / k : i % k) + col0;
     const int tile = interleave >= 0 ? 2 * (r >> 4) + interleave : (r + row0) >> 4;
     const int rr = interleave >= 0 ? r & 15 : (r + row0) & 15;
     dst[((size_t)tile * kt + (c >> 5)) * 512 + (((c & 31) >> 3) * 16 + rr) * 8 + (c & 7)] = src[i];
   }
 }
-int launch_pack(hipStream_t st, const uint16_t* src, int rows, int k, uint16_t* dst, int kt, int row0, int col0, int interleave) {
+int launch_pack(hipStream_t st, const uint16_t* src, int rows, int k, uint16_t* dst, int kt, int row0, int col0, int interleave, bool transpose) {
   const size_t n = (size_t)rows * k;
-  hipLaunchKernelGGL(pack_kernel, dim3((unsigned)((n + 2047) / 2048)), dim3(256), 0, st, src, rows, k, dst, kt, row0, col0, interleave);
+  hipLaunchKernelGGL(pack_kernel, dim3((unsigned)((n + 2047) / 2048)), dim3(256), 0, st, src, rows, k, dst, kt, row0, col0, interleave, (int)transpose);
   return DSK_OK;
 }
 __global__ __launch_bounds__(256) void widen_kernel(const uint16_t* __restrict__ src, float* __restrict__ dst, size_t n) {
@@ -78,6 +78,14 @@ DEV void store_plain(const LinArgs& a, int row, int feature, f32x4 v) {
   if (a.epi == LIN_SOFTCAP) {
 #pragma unroll
     for (int i = 0; i < 4; ++i) v[i] = a.p0 * tanhf(v[i] / a.p0);
+  } else if (a.epi == LIN_SCALE) {
+    v *= a.p0;
+  } else if (a.epi == LIN_XIELU) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = 0.5f * v[i] + (v[i] > 0.f ? a.p0 * v[i] * v[i] : a.p1 * (expm1f(v[i]) - v[i]));
+  } else if (a.epi == LIN_TANH_F && feature >= a.n_wide) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = tanhf(v[i]);
   }
   if (feature < a.n_wide) *reinterpret_cast<four*>(reinterpret_cast<T*>(a.out_t) + (size_t)row * a.ld_t + feature) = to_four<T>(v);
   else *reinterpret_cast<f32x4*>(a.out_f + (size_t)row * a.ld_f + feature - a.n_wide) = v;
@@ -89,6 +97,13 @@ DEV void store_glu(const LinArgs& a, int row, int feature, const f32x4& g, const
 #pragma unroll
   for (int i = 0; i < 4; ++i) v[i] = glu(g[i], u[i], a.p0, a.p1, a.p2);
   *reinterpret_cast<four*>(reinterpret_cast<T*>(a.out_t) + (size_t)row * a.ld_t + feature) = to_four<T>(v);
+}
+
+// the operand a product's features from `feature` on read
+template <typename T>
+DEV const T* operand(const LinArgs& a, int feature) {
+  const T* p = reinterpret_cast<const T*>(a.a_t);
+  return a.a_seg ? p + (size_t)min(feature / a.a_seg, a.a_ops - 1) * a.a_stride : p;
 }
 
 // ---- prompts -------------------------------------------------------------------------------------
@@ -112,7 +127,7 @@ DEV void lin_body(const LinArgs& a, const int* gather, int row0, int n_rows, int
     src_w[i] = reinterpret_cast<const char*>(a.w) + (size_t)rt * a.kt * 1024 + lane * 16;
     int r = min(t * 16 + (lane & 15), n_rows - 1);
     r = gather ? gather[row0 + r] : row0 + r;
-    src_a[i] = reinterpret_cast<const T*>(a.a_t) + (size_t)r * a.lda + (lane >> 4) * 8;
+    src_a[i] = operand<T>(a, f0) + (size_t)r * a.lda + (lane >> 4) * 8;
   }
   auto stage = [&](int kt, char* buf) {
 #pragma unroll
@@ -224,7 +239,7 @@ DEV void few_body(const LinArgs& a, int rt0, int a_row, int out_row, float* lds)
   constexpr int U = 4;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const bf16x8* w0 = reinterpret_cast<const bf16x8*>(a.w) + (size_t)rt0 * a.kt * 64 + lane;
-  const T* x0 = reinterpret_cast<const T*>(a.a_t) + (size_t)a_row * a.lda + (lane >> 4) * 8;
+  const T* x0 = operand<T>(a, rt0 * 16) + (size_t)a_row * a.lda + (lane >> 4) * 8;
   f32x4 acc[NR];
 #pragma unroll
   for (int i = 0; i < NR; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -295,13 +310,14 @@ __global__ __launch_bounds__(256) void few_kernel(const FewArgs f) {
   const LinArgs& a = f.t[i];
   if (i > 0) b -= f.wg_end[i - 1];
   const int row = min(c, a.rows - 1);
-  few_body<T, 1>(a, b, row, c < a.rows ? c : -1, lds);
+  few_body<T, 1>(a, b, a.row_seq ? a.seqs[a.row_seq[row]].row0 : row, c < a.rows ? c : -1, lds);
 }
 
 // ---- launches ------------------------------------------------------------------------------------
 static int lin_lds(bool f32) { return 2 * (16 * 1024 + 16 * 64 * (f32 ? 32 : 16)); }
 static int check_lin(const LinArgs& a, const char* what) {
   if (!a.w || !a.a_t || a.rows < 1 || a.kt < 2 || (a.kt & 1) || a.rt < 1 || a.lda < a.kt * 32) DSK_FAIL(DSK_ERR_INVALID, "%s: rows %d kt %d rt %d lda %d", what, a.rows, a.kt, a.rt, a.lda);
+  if (a.a_seg < 0 || (a.a_seg & 15) || (a.a_seg && a.a_ops < 1)) DSK_FAIL(DSK_ERR_INVALID, "%s: %d features per operand", what, a.a_seg);
   return DSK_OK;
 }
 template <typename K>
@@ -311,6 +327,7 @@ static int allow_lds(K k, int bytes) {
 }
 int launch_lin(hipStream_t st, const LinArgs& a, bool f32) {
   DSK_TRY(check_lin(a, "lin"));
+  if ((a.a_seg & 127) || a.row_seq) DSK_FAIL(DSK_ERR_INVALID, "lin: %d features per operand", a.a_seg);
   const dim3 grid(cdiv(a.rows, 128), cdiv(a.rt, 8));
   const int lds = lin_lds(f32);
   if (f32) {

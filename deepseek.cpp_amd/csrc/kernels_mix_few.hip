@@ -4,6 +4,7 @@
 //               the last of a (sequence, key head)'s workgroups to arrive merges the parts
 //   mLSTM       (sequence, head): gates, one step of the recurrence, norm, output gate
 //   delta rule  (sequence, head): convolution, low-rank second halves, unit norms, decays, one step, norm, output gate
+//   wkv         (sequence, head): low-rank second half and decays, one step with the current token's bonus, norm, output gate
 //   router      one workgroup for the whole step
 // Same formulas and the same roundings to the activation type as the prompt kernels (kernels_chunk_attn.hip, kernels_recur.hip).
 #include "layered_kernels.h"
@@ -371,6 +372,85 @@ DEV void mlstm_few(const MlstmArgs& a, int b, float* lds) {
               reinterpret_cast<T*>(a.out_t) + (size_t)row * a.out_ld + h * a.vdim);
 }
 
+// second half of a low-rank pair out of LDS: 256 rows at a time, four threads per row share its columns; sums in red[4][2 HD].
+// row_of(r): the row of low_w; groups(r, g0, g1): its groups of 8 columns that are not zero
+template <typename T, typename R, typename G>
+DEV void low_rank(const MixFewArgs& f, const float* low, float* red, int nr, R row_of, G groups) {
+  const int tid = threadIdx.x;
+  for (int r0 = 0; r0 < nr; r0 += 256) {
+    const int r = r0 + (tid & 255);
+    if (r >= nr) continue;
+    const int R_ = row_of(r);
+    int g0, g1;
+    groups(r, g0, g1);
+    const bf16* w = reinterpret_cast<const bf16*>(f.low_w) + (size_t)(R_ >> 4) * f.low_kt * 512 + (R_ & 15) * 8;
+    float z = 0.f;
+#pragma unroll 4
+    for (int gr = g0 + (tid >> 8); gr < g1; gr += 4) {
+      float x[8];
+      load8<bf16>(w + (size_t)(gr >> 2) * 512 + (gr & 3) * 128, x);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) z += x[e] * low[gr * 8 + e];
+    }
+    red[(tid >> 8) * 2 * HD + r] = z;
+  }
+}
+DEV float low_sum(const float* red, int r) { return (red[r] + red[2 * HD + r]) + (red[4 * HD + r] + red[6 * HD + r]); }
+
+template <typename T, int RK>
+DEV void wkv_few(const MixFewArgs& f, int b, float* lds) {
+  const WkvArgs& a = f.wkv;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, dim = a.dim;
+  const int h = b % a.heads, row = b / a.heads;
+  const SeqDesc s = a.p.seqs[row];
+  float *r = lds, *k = r + HD, *v = k + HD, *w = v + HD, *o = w + HD, *bonus = o + HD, *low = bonus + 4;
+  float* red = low + f.low_kt * 32;  // [16][HD], before that [4][2 HD]
+  float* S0 = reinterpret_cast<float*>(s.state + a.off_s) + (size_t)h * dim * dim;
+  const HeadTile t = head_tile(dim, dim);
+  float S[RK];
+  load_state<RK>(S0, t, dim, s.pos0 == 0, S);
+  const T* P = reinterpret_cast<const T*>(a.proj_t) + (size_t)row * a.ld + h * dim;
+  for (int i = tid; i < f.low_kt * 32; i += NT) low[i] = i < f.low_a ? f.wkv_low[(size_t)row * f.wkv_low_ld + i] : 0.f;
+  for (int i = tid; i < dim; i += NT) {
+    r[i] = (float)P[a.col_r + i];
+    k[i] = (float)P[a.col_k + i];
+    v[i] = (float)P[a.col_v + i];
+  }
+  __syncthreads();
+  low_rank<T>(f, low, red, dim, [&](int i) { return h * dim + i; }, [&](int, int& g0, int& g1) {
+    g0 = 0;
+    g1 = (f.low_a + 7) >> 3;
+  });
+  if (wave == NW - 1) {
+    float z = 0.f;
+    for (int i = lane; i < dim; i += 64) z += r[i] * a.u[h * dim + i] * k[i];
+    z = wave_sum(z);
+    if (lane == 0) bonus[0] = z;
+  }
+  __syncthreads();
+  for (int i = tid; i < dim; i += NT) w[i] = expf(-expf(low_sum(red, i) + a.w0[h * dim + i]));
+  __syncthreads();
+  float z = 0.f;
+  const float vc = t.on ? v[t.col] : 0.f;
+#pragma unroll
+  for (int i = 0; i < RK; ++i)
+    if (i < t.kn) {
+      z += S[i] * r[t.k0 + i];
+      S[i] = w[t.k0 + i] * S[i] + k[t.k0 + i] * vc;
+    }
+  store_state<RK>(S0, t, dim, S);
+  const int per = (dim + t.parts - 1) / t.parts, used = (dim + per - 1) / per;
+  if (t.on && t.kn) red[(size_t)(t.k0 / per) * HD + t.col] = z;
+  __syncthreads();
+  if (tid < dim) {
+    float sum = bonus[0] * v[tid];
+    for (int i = 0; i < used; ++i) sum += red[(size_t)i * HD + tid];
+    o[tid] = sum;
+  }
+  __syncthreads();
+  head_out<T>(o, dim, a.eps, a.out_norm + h * dim, [&](int i) { return silu_f((float)P[a.col_g + i]); }, reinterpret_cast<T*>(a.out_t) + (size_t)row * a.out_ld + h * dim);
+}
+
 template <typename T, int RK>
 DEV void delta_few(const MixFewArgs& f, int b, float* lds) {
   const DeltaArgs& a = f.delta;
@@ -407,25 +487,12 @@ DEV void delta_few(const MixFewArgs& f, int b, float* lds) {
     }
   }
   __syncthreads();
-  // low-rank second halves: 256 rows at a time, four threads per row share its columns
-  const int nr = dim + vdim;
-  for (int r0 = 0; r0 < nr; r0 += 256) {
-    const int r = r0 + (tid & 255);
-    if (r < nr) {
-      const int R = r < dim ? h * dim + r : a.heads * dim + h * vdim + r - dim;
-      const int g0 = r < dim ? 0 : f.low_a >> 3, g1 = r < dim ? (f.low_a + 7) >> 3 : (f.low_a + f.low_g + 7) >> 3;
-      const bf16* w = reinterpret_cast<const bf16*>(f.low_w) + (size_t)(R >> 4) * f.low_kt * 512 + (R & 15) * 8;
-      float z = 0.f;
-#pragma unroll 4
-      for (int gr = g0 + (tid >> 8); gr < g1; gr += 4) {
-        float x[8];
-        load8<bf16>(w + (size_t)(gr >> 2) * 512 + (gr & 3) * 128, x);
-#pragma unroll
-        for (int e = 0; e < 8; ++e) z += x[e] * low[gr * 8 + e];
-      }
-      red[(tid >> 8) * 2 * HD + r] = z;
-    }
-  }
+  const int nr = a.head_decay ? 0 : dim + vdim;
+  low_rank<T>(f, low, red, nr, [&](int r) { return r < dim ? h * dim + r : a.heads * dim + h * vdim + r - dim; },
+              [&](int r, int& g0, int& g1) {
+                g0 = r < dim ? 0 : f.low_a >> 3;
+                g1 = r < dim ? (f.low_a + 7) >> 3 : (f.low_a + f.low_g + 7) >> 3;
+              });
   if (wave < 3) {  // |q|^2, |k|^2, k . q
     const float *x = wave == 0 ? q : k, *y = wave == 1 ? k : q;
     float ss = 0.f;
@@ -436,9 +503,14 @@ DEV void delta_few(const MixFewArgs& f, int b, float* lds) {
   __syncthreads();
   const float qr = a.q_scale / sqrtf(sc[0] + a.unit_eps), kr = 1.f / sqrtf(sc[1] + a.unit_eps);
   for (int r = tid; r < nr; r += NT) {
-    const float z = (red[r] + red[2 * HD + r]) + (red[4 * HD + r] + red[6 * HD + r]);
+    const float z = low_sum(red, r);
     if (r < dim) g[r] = expf(-a.a_rate[h] * softplus_f(z + a.dt_bias[h * dim + r]));
     else gate[r - dim] = sigmoid_f(z);
+  }
+  if (a.head_decay) {
+    const float d = expf(-a.a_rate[h] * softplus_f(a.gate_f[(size_t)row * a.ld_gate + a.col_a + h] + a.dt_bias[h]));
+    for (int r = tid; r < dim; r += NT) g[r] = d;
+    for (int r = tid; r < vdim; r += NT) gate[r] = silu_f((float)P[a.col_g + h * vdim + r]);
   }
   const float beta = sigmoid_f(a.gate_f[(size_t)row * a.ld_gate + a.col_b + h]);
   __syncthreads();
@@ -491,6 +563,13 @@ __global__ __launch_bounds__(NT) void mix_few_kernel(const MixFewArgs f) {
     }
     b -= f.rows * f.mlstm.heads;
   }
+  if (f.has_wkv) {
+    if (b < f.rows * f.wkv.heads) {
+      wkv_few<T, RK>(f, b, lds);
+      return;
+    }
+    b -= f.rows * f.wkv.heads;
+  }
   if (f.has_route) {
     if (b == 0) {
       route_few_body(f.moe, reinterpret_cast<char*>(lds));
@@ -507,6 +586,7 @@ static size_t mix_lds(const MixFewArgs& f) {
   if (f.has_attn) n = std::max(n, attn_few_lds(f.attn));
   if (f.has_mlstm) n = std::max(n, (size_t)(4 + NW) * HD * 4);
   if (f.has_delta) n = std::max(n, ((size_t)(6 + 2 * NW) * HD + 4 + f.low_kt * 32) * 4);
+  if (f.has_wkv) n = std::max(n, ((size_t)(5 + NW) * HD + 4 + f.low_kt * 32) * 4);
   return n;
 }
 bool mix_few_fits(const MixFewArgs& f) {
@@ -514,13 +594,14 @@ bool mix_few_fits(const MixFewArgs& f) {
   if (f.has_attn && 2 * f.attn.heads / f.attn.kv_heads * f.splits > NW * 4 * f.attn.vdim_p) return false;  // (the merge's sums in LDS)
   if (f.has_mlstm && (f.mlstm.dim > HD || f.mlstm.vdim > HD)) return false;
   if (f.has_delta && (f.delta.dim > HD || f.delta.vdim > HD)) return false;
+  if (f.has_wkv && f.wkv.dim > HD) return false;
   if (f.has_route && (f.moe.experts > ROUTE_MAX_EXPERTS || f.moe.top + f.moe.shared > 64)) return false;
   return f.rows <= 16 && mix_lds(f) <= 128 * 1024;
 }
 template <typename T, int RK>
 static int mix_t(hipStream_t st, const MixFewArgs& f) {
   const size_t lds = mix_lds(f);
-  const int grid = f.rows * ((f.has_delta ? f.delta.heads : 0) + (f.has_mlstm ? f.mlstm.heads : 0) + (f.has_attn ? f.attn.kv_heads * f.splits : 0)) + (f.has_route ? 1 : 0);
+  const int grid = f.rows * ((f.has_delta ? f.delta.heads : 0) + (f.has_mlstm ? f.mlstm.heads : 0) + (f.has_wkv ? f.wkv.heads : 0) + (f.has_attn ? f.attn.kv_heads * f.splits : 0)) + (f.has_route ? 1 : 0);
   auto k = mix_few_kernel<T, RK>;
   HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
   hipLaunchKernelGGL(k, dim3(grid), dim3(NT), lds, st, f);
@@ -531,6 +612,7 @@ static int mix_rk(hipStream_t st, const MixFewArgs& f) {
   int rk = 1;
   if (f.has_mlstm) rk = std::max(rk, head_rk(f.mlstm.dim, f.mlstm.vdim));
   if (f.has_delta) rk = std::max(rk, head_rk(f.delta.dim, f.delta.vdim));
+  if (f.has_wkv) rk = std::max(rk, head_rk(f.wkv.dim, f.wkv.dim));
   return rk <= 8 ? mix_t<T, 8>(st, f) : rk <= 16 ? mix_t<T, 16>(st, f) : rk <= 32 ? mix_t<T, 32>(st, f) : mix_t<T, 64>(st, f);
 }
 int launch_mix_few(hipStream_t st, const MixFewArgs& f, bool f32) {

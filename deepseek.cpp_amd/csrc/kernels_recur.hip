@@ -1,5 +1,5 @@
-// kernels_recur.hip -- recurrent mixers of layered models: the gated delta rule with a decay per key channel, and mLSTM's matrix
-// memory.  Everything that enters the recurrence is computed in 32-bit; the state is 32-bit and lives in the sequence's arena.
+// kernels_recur.hip -- recurrent mixers of layered models: the gated delta rule with a decay per key channel or per head, mLSTM's
+// matrix memory, and time mixing with a bonus for the current token (wkv).  Everything that enters the recurrence is computed in 32-bit; the state is 32-bit and lives in the sequence's arena.
 //
 // The columns of a head's state S [dim][vdim] never meet each other inside the recurrence, so a scan cuts a head into slices of 16
 // columns: one workgroup of 4 waves per (slice, head, sequence), a wave holds 4 columns, 16 lanes share a column's dim key channels
@@ -28,7 +28,9 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(const DeltaArgs a) {
   if (unit >= 2 * a.kv_heads + a.heads) {
     const int h = unit - 2 * a.kv_heads - a.heads;
     const float rate = a.a_rate[h];
-    for (int i = lane; i < a.dim; i += 64) {
+    if (a.head_decay) {
+      if (lane < n_rows) a.g[(row0 + lane) * a.heads + h] = expf(-rate * softplus_f(a.gate_f[(row0 + lane) * a.ld_gate + a.col_a + h] + a.dt_bias[h]));
+    } else for (int i = lane; i < a.dim; i += 64) {
       const float bias = a.dt_bias[h * a.dim + i];
 #pragma unroll 4
       for (int t = 0; t < n_rows; ++t)
@@ -142,7 +144,7 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const DeltaArgs a) {
       const bool in = ok && lk + i < dim;
       rq[i] = in ? a.q[row * nq + (size_t)kv * dim + lk + i] : 0.f;
       rk[i] = in ? a.k[row * nq + (size_t)kv * dim + lk + i] : 0.f;
-      rg[i] = in ? a.g[row * a.heads * dim + (size_t)h * dim + lk + i] : 0.f;
+      rg[i] = in ? (a.head_decay ? a.g[row * a.heads + h] : a.g[row * a.heads * dim + (size_t)h * dim + lk + i]) : 0.f;
     }
     const int c = blockIdx.x * 16 + (tid & 15);
     rv = ok && c < a.vdim ? a.v[row * nv + (size_t)h * a.vdim + c] : 0.f;
@@ -236,8 +238,8 @@ int launch_delta_scan(hipStream_t st, const DeltaArgs& a) {
   }, "delta");
 }
 
-// ---- behind a recurrence: per-head RMS norm, weight, sigmoid gate ------------------------------------
-// value(h, i): element i of head h; gate(c), w[c or i]: by place among all heads or inside one
+// ---- behind a recurrence: per-head RMS norm, weight, gate ---------------------------------------------
+// value(h, i): element i of head h; gate(c): the factor; w[c or i]: by place among all heads or inside one
 template <typename T, typename V, typename G>
 DEV void head_norm_gate(V value, int heads, int vdim, float eps, const float* w, bool shared_w, G gate, T* out) {
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -252,7 +254,7 @@ DEV void head_norm_gate(V value, int heads, int vdim, float eps, const float* w,
 #pragma unroll
     for (int i = 0; i < RECUR_MAX_DIM / 64; ++i) {
       const int e = lane + 64 * i, c = h * vdim + e;
-      if (e < vdim) out[c] = (T)(v[i] * r * w[shared_w ? e : c] * sigmoid_f(gate(c)));
+      if (e < vdim) out[c] = (T)(v[i] * r * w[shared_w ? e : c] * gate(c));
     }
   }
 }
@@ -260,8 +262,9 @@ template <typename T>
 __global__ __launch_bounds__(256) void delta_out_kernel(const DeltaArgs a) {
   const size_t row = blockIdx.x;
   const float *gl = a.low_f + row * a.ld_low + (size_t)a.heads * a.dim, *o = a.o + row * a.heads * a.vdim;
-  head_norm_gate<T>([&](int h, int i) { return o[h * a.vdim + i]; }, a.heads, a.vdim, a.eps, a.out_norm, true, [&](int c) { return gl[c]; },
-                    reinterpret_cast<T*>(a.out_t) + row * a.out_ld);
+  const T* gp = reinterpret_cast<const T*>(a.proj_t) + row * a.ld + a.col_g;
+  head_norm_gate<T>([&](int h, int i) { return o[h * a.vdim + i]; }, a.heads, a.vdim, a.eps, a.out_norm, true,
+                    [&](int c) { return a.silu_gate ? silu_f((float)gp[c]) : sigmoid_f(gl[c]); }, reinterpret_cast<T*>(a.out_t) + row * a.out_ld);
 }
 int launch_delta_out(hipStream_t st, const DeltaArgs& a, bool f32) {
   if (f32) hipLaunchKernelGGL(delta_out_kernel<float>, dim3(a.p.rows), dim3(256), 0, st, a);
@@ -277,7 +280,7 @@ __global__ __launch_bounds__(256) void mlstm_out_kernel(const MlstmArgs a, const
   head_norm_gate<T>([&](int h, int i) {
     const float v = o[h * ld + i];
     return RAW ? v / (fmaxf(fabsf(o[h * ld + a.vdim]), floor_[row * a.heads + h]) + a.floor_eps) : v;
-  }, a.heads, a.vdim, a.eps, a.out_norm, false, [&](int c) { return (float)gl[c]; }, reinterpret_cast<T*>(a.out_t) + row * a.out_ld);
+  }, a.heads, a.vdim, a.eps, a.out_norm, false, [&](int c) { return sigmoid_f((float)gl[c]); }, reinterpret_cast<T*>(a.out_t) + row * a.out_ld);
 }
 int launch_mlstm_out(hipStream_t st, const MlstmArgs& a, const ChunkScan* c, bool f32) {
   if (a.vdim > RECUR_MAX_DIM) DSK_FAIL(DSK_ERR_UNSUPPORTED, "mlstm: value size %d (max %d)", a.vdim, (int)RECUR_MAX_DIM);
@@ -429,3 +432,101 @@ static int mlstm_t(hipStream_t st, const MlstmArgs& a) {
   }, "mlstm");
 }
 int launch_mlstm_scan(hipStream_t st, const MlstmArgs& a, bool f32) { return f32 ? mlstm_t<float>(st, a) : mlstm_t<bf16>(st, a); }
+
+// ---- wkv: the scan -----------------------------------------------------------------------------------
+template <typename T, int KPL>
+__global__ __launch_bounds__(256) void wkv_scan_kernel(const WkvArgs a) {
+  constexpr int DK = 16 * KPL;
+  __shared__ __attribute__((aligned(16))) float sr_[SCAN_CH][DK], sk_[SCAN_CH][DK], sw_[SCAN_CH][DK];
+  __shared__ float sv_[SCAN_CH][16], sbonus[SCAN_CH];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int kl = lane & 15, vl = wave * 4 + (lane >> 4);
+  const int h = blockIdx.y, dim = a.dim, n_all = a.heads * dim;
+  const int col = blockIdx.x * 16 + vl;
+  const bool live = col < dim;
+  const SeqDesc s = a.p.seqs[blockIdx.z];
+  float* S0 = reinterpret_cast<float*>(s.state + a.off_s) + (size_t)h * dim * dim;
+  float S[KPL];
+#pragma unroll
+  for (int i = 0; i < KPL; ++i) {
+    const int k = kl * KPL + i;
+    S[i] = s.pos0 > 0 && live && k < dim ? S0[(size_t)k * dim + col] : 0.f;
+  }
+  const int lt = tid >> 4, lk = (tid & 15) * KPL;
+  float rr[KPL], rk[KPL], rw[KPL], rv = 0.f, rb = 0.f;
+  auto fetch = [&](int t0) {
+    const int t = t0 + lt;
+    const bool ok = t < s.len;
+    const size_t row = (size_t)(s.row0 + (ok ? t : 0));
+    const T* P = reinterpret_cast<const T*>(a.proj_t) + row * a.ld + h * dim;
+    rb = 0.f;
+#pragma unroll
+    for (int i = 0; i < KPL; ++i) {
+      const bool in = ok && lk + i < dim;
+      rr[i] = in ? (float)P[a.col_r + lk + i] : 0.f;
+      rk[i] = in ? (float)P[a.col_k + lk + i] : 0.f;
+      rw[i] = in ? expf(-expf(a.low_f[row * a.ld_low + h * dim + lk + i] + a.w0[h * dim + lk + i])) : 0.f;
+      rb += in ? rr[i] * a.u[h * dim + lk + i] * rk[i] : 0.f;
+    }
+    rb = row_sum(rb);
+    const int c = blockIdx.x * 16 + (tid & 15);
+    rv = ok && c < dim ? (float)P[a.col_v + c] : 0.f;
+  };
+  fetch(0);
+  for (int t0 = 0; t0 < s.len; t0 += SCAN_CH) {
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < KPL; ++i) {
+      sr_[lt][lk + i] = rr[i];
+      sk_[lt][lk + i] = rk[i];
+      sw_[lt][lk + i] = rw[i];
+    }
+    sv_[lt][tid & 15] = rv;
+    if ((tid & 15) == 0) sbonus[lt] = rb;
+    __syncthreads();
+    if (t0 + SCAN_CH < s.len) fetch(t0 + SCAN_CH);
+    const int n = min((int)SCAN_CH, s.len - t0);
+    for (int t = 0; t < n; ++t) {
+      const float v = sv_[t][vl];
+      float o = 0.f;
+#pragma unroll
+      for (int i = 0; i < KPL; ++i) {
+        o += S[i] * sr_[t][kl * KPL + i];
+        S[i] = sw_[t][kl * KPL + i] * S[i] + sk_[t][kl * KPL + i] * v;
+      }
+      o = row_sum(o);
+      if (kl == 0 && live) a.o[(size_t)(s.row0 + t0 + t) * n_all + h * dim + col] = o + sbonus[t] * v;
+    }
+  }
+  if (live)
+#pragma unroll
+    for (int i = 0; i < KPL; ++i) {
+      const int k = kl * KPL + i;
+      if (k < dim) S0[(size_t)k * dim + col] = S[i];
+    }
+}
+template <typename T>
+static int wkv_t(hipStream_t st, const WkvArgs& a) {
+  return by_kpl(a, [&](int kpl) {
+    const dim3 grid(cdiv(a.dim, 16), a.heads, a.p.n_seqs);
+    if (kpl == 2) hipLaunchKernelGGL((wkv_scan_kernel<T, 2>), grid, dim3(256), 0, st, a);
+    else if (kpl == 4) hipLaunchKernelGGL((wkv_scan_kernel<T, 4>), grid, dim3(256), 0, st, a);
+    else if (kpl == 8) hipLaunchKernelGGL((wkv_scan_kernel<T, 8>), grid, dim3(256), 0, st, a);
+    else hipLaunchKernelGGL((wkv_scan_kernel<T, 16>), grid, dim3(256), 0, st, a);
+    return (int)DSK_OK;
+  }, "wkv");
+}
+int launch_wkv_scan(hipStream_t st, const WkvArgs& a, bool f32) { return f32 ? wkv_t<float>(st, a) : wkv_t<bf16>(st, a); }
+template <typename T>
+__global__ __launch_bounds__(256) void wkv_out_kernel(const WkvArgs a) {
+  const size_t row = blockIdx.x;
+  const float* o = a.o + row * a.heads * a.dim;
+  const T* gp = reinterpret_cast<const T*>(a.proj_t) + row * a.ld + a.col_g;
+  head_norm_gate<T>([&](int h, int i) { return o[h * a.dim + i]; }, a.heads, a.dim, a.eps, a.out_norm, false, [&](int c) { return silu_f((float)gp[c]); },
+                    reinterpret_cast<T*>(a.out_t) + row * a.out_ld);
+}
+int launch_wkv_out(hipStream_t st, const WkvArgs& a, bool f32) {
+  if (f32) hipLaunchKernelGGL(wkv_out_kernel<float>, dim3(a.p.rows), dim3(256), 0, st, a);
+  else hipLaunchKernelGGL(wkv_out_kernel<bf16>, dim3(a.p.rows), dim3(256), 0, st, a);
+  return DSK_OK;
+}

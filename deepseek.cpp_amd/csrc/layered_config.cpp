@@ -101,6 +101,35 @@ DeltaSpec parse_delta(const Obj& o, const std::string& name) {
   check_groups(o, a.heads, a.kv_heads);
   return a;
 }
+WkvSpec parse_wkv(const Obj& o, const std::string& name) {
+  WkvSpec a;
+  a.name = name;
+  a.heads = o.size("heads");
+  a.dim = o.size("dim");
+  return a;
+}
+LatentSpec parse_latent(const Obj& o, const std::string& name) {
+  LatentSpec a;
+  a.name = name;
+  a.heads = o.size("heads");
+  a.dim = o.size("dim");
+  a.rot_dim = o.size("rot_dim");
+  a.vdim = o.size("vdim");
+  a.q_rank = o.size("q_rank");
+  a.kv_rank = o.size("kv_rank");
+  a.window = o.at("mask").size("size");
+  a.scale = o.num("scale");
+  a.rot = parse_rot(o.at("rot"));
+  if (o.bad->empty() && a.rot.dims > a.rot_dim) o.fail("rotates more dimensions than 'rot_dim'");
+  return a;
+}
+DenseSpec parse_dense(const Obj& o, const std::string& name) {
+  DenseSpec d;
+  d.name = name;
+  if (o.str("kind") != "dense") o.fail("'kind' is not known");
+  d.ff = o.size("ff");
+  return d;
+}
 MoeSpec parse_moe(const Obj& o, const std::string& name) {
   MoeSpec m;
   m.name = name;
@@ -163,11 +192,63 @@ void parse_timerax(const Obj& root, LayeredSpec* s) {
   }
 }
 
+// Ranutar: sandwich layers (a norm with its weight around zero before and behind each sublayer, a causal convolution in front of it)
+// of three kinds - "wkv" (time mixing), "delta" (gated delta rule, a decay per head), "latent_attention" (sliding window) - and dense
+// feed-forwards.
+void parse_ranutar(const Obj& root, LayeredSpec* s) {
+  s->width = root.size("width");
+  s->vocab = root.size("vocab");
+  s->eps = root.at("norm").num("eps");
+  s->norm_offset = 1.0;
+  s->logit_scale = root.num("logit_scale");
+  s->embed = "embed";
+  s->final_norm = "final.norm";
+  s->head = "head";
+  const int taps = root.at("canon").size("taps");
+  const JVal* layers = root.v->get("layers");
+  if (!layers || layers->kind != JVal::ARR || layers->arr.empty()) {
+    root.fail("lists no layers");
+    return;
+  }
+  for (size_t i = 0; i < layers->arr.size(); ++i) {
+    const Obj o(&layers->arr[i], root.path + ".layers[" + std::to_string(i) + "]", root.bad);
+    LayerSpec l;
+    const std::string pre = "l" + std::to_string(i) + ".", type = o.str("type");
+    l.sandwich = true;
+    l.taps = taps;
+    l.norm = pre + "norm1";
+    l.post = pre + "norm1b";
+    l.conv = pre + "canon1";
+    const Obj mix = o.at("mixer");
+    if (type == "wkv") {
+      l.has_wkv = true;
+      l.wkv = parse_wkv(mix, pre + "mix");
+    } else if (type == "delta") {
+      l.has_delta = true;
+      l.delta = parse_delta(mix, pre + "mix");
+      l.delta.head_decay = l.delta.silu_gate = true;
+    } else if (type == "latent_attention") {
+      l.has_latent = true;
+      l.latent = parse_latent(mix, pre + "mix");
+    } else {
+      o.fail("has the unknown type '" + type + "'");
+    }
+    if (o.has("mlp")) {
+      l.has_dense = true;
+      l.dense = parse_dense(o.at("mlp"), pre + "mlp");
+      l.ff_norm = pre + "norm2";
+      l.ff_post = pre + "norm2b";
+      l.ff_conv = pre + "canon2";
+    }
+    s->layers.push_back(l);
+  }
+}
+
 struct Design {
   const char* name;
   void (*parse)(const Obj& root, LayeredSpec* out);
 };
-const Design DESIGNS[] = {{"Timerax", parse_timerax}};
+const Design DESIGNS[] = {{"Timerax", parse_timerax}, {"Ranutar", parse_ranutar}};
 
 }  // namespace
 

@@ -1,9 +1,10 @@
 // layered_model.cpp -- layered models (layered.h) behind the model-family table: weights into HBM, the sequences' state, steps.
 //
-// A layer is five launches and its mixers': [residual sum + norm] -> one matrix product for everything that reads the norm (the
-// mixers' projections, gates, the router) -> mixers -> their output products -> experts (up, down).  A step's tokens are packed
-// without padding; every sequence owns an arena whose size does not depend on its length (one chunk of keys and values,
-// recurrent state, convolution inputs).  Steps of at most 16 single tokens run on the kernels for few rows, from a captured graph.
+// A parallel layer is five launches and its mixers': [residual sum + norm] -> one matrix product for everything that reads the norm
+// (the mixers' projections, gates, the router) -> mixers -> their output products -> experts (up, down).  A sandwich layer has a second
+// [residual sum + norms + convolution] between its mixer and a dense feed-forward.  A step's tokens are packed without padding; every
+// sequence owns an arena whose size does not depend on its length (one chunk of keys and values, a window of latents, recurrent
+// state, convolution inputs).  Steps of at most 16 single tokens run on the kernels for few rows, from a captured graph.
 #include "layered.h"
 
 #include <math.h>
@@ -18,8 +19,15 @@ enum { FEW = 16, LOGIT_ROWS = 128 };
 
 size_t up(size_t v, size_t a) { return (v + a - 1) / a * a; }
 
+struct ConvW {           // a sandwich layer's convolution in front of a sublayer
+  float *w = nullptr, *mu = nullptr;
+  int n_mix = 0;         // blends with the previous token (wkv), in the order of the projections
+  size_t off_in = 0, off_prev = 0;
+};
 struct LayerW {
   float* norm = nullptr;
+  float *post = nullptr, *ff_norm = nullptr, *ff_post = nullptr;
+  ConvW conv, ff_conv;
   PackedMat proj;        // every product of the norm's output: wide segments (activation type), then 32-bit segments
   int n_wide = 0;        // columns of the wide part (multiple of 64)
   // attention
@@ -39,6 +47,21 @@ struct LayerW {
   PackedMat d_low2, d_o;  // both second halves of the low-rank pairs, block-diagonal
   float *d_conv = nullptr, *d_rate = nullptr, *d_dt = nullptr, *d_norm = nullptr;
   size_t off_ds = 0, off_dc = 0;
+  int d_a = 0, d_g = 0;   // (decay per head, gate by silu)
+  // wkv
+  int w_r = 0, w_k = 0, w_v = 0, w_g = 0, w_low = 0, seg = 0;  // seg: features per blend
+  PackedMat w_low2, w_o;
+  float *w_w0 = nullptr, *w_u = nullptr, *w_norm = nullptr;
+  size_t off_ws = 0;
+  // latent attention
+  int l_q = 0, l_kv = 0;
+  int dim_p = 0, rot_p = 0, vdim_p = 0, rank_p = 0;
+  float *l_qn = nullptr, *l_kvn = nullptr;
+  PackedMat l_uq, l_ukv, l_abs, l_o;  // l_abs: W_uk transposed per head, queries into the latent space
+  size_t off_lc = 0;
+  // dense feed-forward
+  PackedMat ff_up, ff_down;
+  float ff_pos = 0.f, ff_neg = 0.f;
   float *pair_a = nullptr, *pair_b = nullptr;
   int router = 0;
   ExpertMat e_up{}, e_down{};
@@ -54,7 +77,7 @@ struct Seq {
 struct DescBuf {
   char *host = nullptr, *dev = nullptr;
   int cap = 0;
-  size_t o_tok = 0, o_row = 0, o_want = 0, o_tile = 0, o_chunk = 0, bytes = 0;
+  size_t o_tok = 0, o_row = 0, o_want = 0, o_tile = 0, o_chunk = 0, o_single = 0, bytes = 0;
 };
 
 struct Graph {
@@ -86,6 +109,10 @@ struct LayeredModel : ModelHead {
   float* x = nullptr;
   char *h = nullptr, *hw = nullptr, *wide = nullptr, *out_a = nullptr, *out_b = nullptr, *qb = nullptr, *kb = nullptr, *vb = nullptr, *hidden = nullptr, *y = nullptr;
   float *narrow = nullptr, *mix_a = nullptr, *mix_b = nullptr, *low = nullptr, *dq = nullptr, *dk = nullptr, *dv = nullptr, *dg = nullptr, *db = nullptr, *o = nullptr;
+  // sandwich layers, latent attention
+  float *h_f = nullptr, *turn = nullptr, *lat_part = nullptr, *lat_ml = nullptr;
+  char *cq = nullptr, *lq = nullptr, *lat = nullptr, *kv = nullptr, *qabs = nullptr;
+  int mixes = 1, lq_ld = 0, max_window = 0, key_cap = 0;  // mixes: blends of h; key_cap: rows of the key workspace
   float *weight = nullptr, *logits = nullptr, *trace_x = nullptr, *sample_scratch = nullptr;
   int *slot_pos = nullptr, *chosen = nullptr, *count = nullptr, *cursor = nullptr, *slot_row = nullptr, *tiles = nullptr, *n_tiles = nullptr, *active = nullptr,
       *active_slot = nullptr, *n_active = nullptr, *next_dev = nullptr;
@@ -100,7 +127,7 @@ struct LayeredModel : ModelHead {
   float* attn_part = nullptr;       // parts of attention outputs (kernels_mix_few.hip)
   unsigned* attn_arrived = nullptr;
   int splits = 1;                   // attention workgroups per (sequence, key head) of the current decode step: a power of two
-  long long fused_layers = 0;       // layers enqueued with the fused decode launch
+  long long fused_layers = 0;       // layers enqueued with the fused decode launches
   std::map<int, Graph> graphs;
   int graph_steps = 0;
   size_t elem() const { return f32 ? 4 : 2; }
@@ -192,6 +219,15 @@ struct Weights {
     DSK_TRY(get(name, rows, k, &p));
     return launch_pack(m->ctx->stream, p, rows, k, dst.w, dst.kt, row0, col0, -1);
   }
+  // heads of `rows` rows behind each other, head i's at dst row row0 + i * stride, from row `first` of its `all` rows on; transpose: the
+  // head's columns become rows
+  int pack_heads(const std::string& name, int heads, int all, int first, int rows, int k, const PackedMat& dst, int row0, int stride, bool transpose = false) {
+    uint16_t* p;
+    DSK_TRY(get(name, heads * all, k, &p));
+    for (int i = 0; i < heads; ++i)
+      DSK_TRY(launch_pack(m->ctx->stream, p + ((size_t)i * all + first) * k, rows, k, dst.w, dst.kt, row0 + i * stride, 0, -1, transpose));
+    return DSK_OK;
+  }
   int matrix(const std::string& name, int rows, int k, PackedMat* dst) {
     DSK_TRY(alloc(dst, rows, k));
     return pack(name, rows, k, *dst, 0);
@@ -276,24 +312,52 @@ int load_layer(Weights& W, LayeredModel* m, const LayerSpec& l, LayerW& w) {
     w.d_q = wide.add(a.name + ".q", a.kv_heads * a.dim, 16);
     w.d_k = wide.add(a.name + ".k", a.kv_heads * a.dim, 16);
     w.d_v = wide.add(a.name + ".v", a.heads * a.vdim, 16);
-    DSK_TRY(W.rows_of(a.name + ".a1", a.dim, &low_a));
-    DSK_TRY(W.rows_of(a.name + ".g1", a.dim, &low_g));
-    w.d_low = wide.add(a.name + ".a1", low_a, 64);  // both, behind each other, are one operand of the second product
-    wide.add(a.name + ".g1", low_g, 1);
+    if (a.head_decay) {
+      w.d_a = narrow.add(a.name + ".a", a.heads, 1);
+    } else {
+      DSK_TRY(W.rows_of(a.name + ".a1", a.dim, &low_a));
+      w.d_low = wide.add(a.name + ".a1", low_a, 64);  // both, behind each other, are one operand of the second product
+    }
+    if (a.silu_gate) {
+      w.d_g = wide.add(a.name + ".g", a.heads * a.vdim, 16);
+    } else {
+      DSK_TRY(W.rows_of(a.name + ".g1", a.dim, &low_g));
+      wide.add(a.name + ".g1", low_g, 1);
+    }
     w.d_b = narrow.add(a.name + ".b", a.heads, 1);
+  }
+  if (l.has_wkv) {
+    const WkvSpec& a = l.wkv;
+    const int n = a.heads * a.dim;
+    w.seg = (int)up(n, 128);  // every projection reads a blend of its own: one operand per `seg` features
+    w.w_r = wide.add(a.name + ".r", n, w.seg);
+    w.w_k = wide.add(a.name + ".k", n, w.seg);
+    w.w_v = wide.add(a.name + ".v", n, w.seg);
+    w.w_g = wide.add(a.name + ".g", n, w.seg);
+    wide.next = 4 * w.seg;
+    DSK_TRY(W.rows_of(a.name + ".w1", std::min(64, a.dim), &low_a));
+    w.w_low = narrow.add(a.name + ".w1", low_a, 1);
+    narrow.next = (int)up(low_a, 64);  // (an operand of the second product as it is)
+  }
+  if (l.has_latent) {
+    const LatentSpec& a = l.latent;
+    w.l_q = narrow.add(a.name + ".dq", a.q_rank, 1);
+    w.l_kv = narrow.add(a.name + ".dkv", a.kv_rank + a.rot_dim, 1);
   }
   if (l.has_moe) w.router = narrow.add(l.moe.name + ".router", l.moe.experts, 1);
   w.n_wide = (int)up(wide.next, 64);
   DSK_TRY(W.alloc(&w.proj, w.n_wide + narrow.next, D));
   for (auto& p : wide.parts) DSK_TRY(W.pack(p.name, p.rows, D, w.proj, p.col));
   for (auto& p : narrow.parts) DSK_TRY(W.pack(p.name, p.rows, D, w.proj, w.n_wide + p.col));
-  if (l.has_attn) {
-    const AttnSpec& a = l.attn;
+  if (l.has_attn || l.has_latent) {
     std::vector<float> f;
-    rot_frequencies(a.rot, &f, &w.rot_amp);
+    rot_frequencies(l.has_attn ? l.attn.rot : l.latent.rot, &f, &w.rot_amp);
     DSK_TRY(dev_alloc_n(m, &w.freq, f.size(), true));
     HIP_TRY(hipStreamSynchronize(m->ctx->stream));
     if (!f.empty()) HIP_TRY(hipMemcpy(w.freq, f.data(), f.size() * 4, hipMemcpyHostToDevice));
+  }
+  if (l.has_attn) {
+    const AttnSpec& a = l.attn;
     DSK_TRY(W.matrix(a.name + ".o", D, a.heads * a.vdim, &w.a_o));
   }
   if (l.has_mlstm) {
@@ -312,12 +376,65 @@ int load_layer(Weights& W, LayeredModel* m, const LayerSpec& l, LayerW& w) {
     DSK_TRY(W.floats_at(a.name + ".v.conv", nv, a.taps, w.d_conv + (size_t)2 * nq * a.taps));
     DSK_TRY(W.floats(a.name + ".A_log", 0, a.heads, &w.d_rate));  // exp() of it below
     DSK_TRY(launch_exp(m->ctx->stream, w.d_rate, a.heads));
-    DSK_TRY(W.floats(a.name + ".dt_bias", 0, a.heads * a.dim, &w.d_dt));
+    DSK_TRY(W.floats(a.name + ".dt_bias", 0, a.head_decay ? a.heads : a.heads * a.dim, &w.d_dt));
     DSK_TRY(W.floats(a.name + ".norm", 0, a.vdim, &w.d_norm));
-    DSK_TRY(W.alloc(&w.d_low2, a.heads * (a.dim + a.vdim), low_a + low_g));
-    DSK_TRY(W.pack(a.name + ".a2", a.heads * a.dim, low_a, w.d_low2, 0, 0));
-    DSK_TRY(W.pack(a.name + ".g2", a.heads * a.vdim, low_g, w.d_low2, a.heads * a.dim, low_a));
+    if (!a.head_decay) {
+      DSK_TRY(W.alloc(&w.d_low2, a.heads * (a.dim + a.vdim), low_a + low_g));
+      DSK_TRY(W.pack(a.name + ".a2", a.heads * a.dim, low_a, w.d_low2, 0, 0));
+      DSK_TRY(W.pack(a.name + ".g2", a.heads * a.vdim, low_g, w.d_low2, a.heads * a.dim, low_a));
+    }
     DSK_TRY(W.matrix(a.name + ".o", D, nv, &w.d_o));
+  }
+  if (l.has_wkv) {
+    const WkvSpec& a = l.wkv;
+    const int n = a.heads * a.dim;
+    DSK_TRY(W.matrix(a.name + ".w2", n, low_a, &w.w_low2));
+    DSK_TRY(W.floats(a.name + ".w0", 0, n, &w.w_w0));
+    DSK_TRY(W.floats(a.name + ".u", a.heads, a.dim, &w.w_u));
+    DSK_TRY(W.floats(a.name + ".norm", 0, n, &w.w_norm));
+    DSK_TRY(W.matrix(a.name + ".o", D, n, &w.w_o));
+    const char* blends[] = {"r", "k", "v", "g", "w"};  // (as the columns of the projection)
+    w.conv.n_mix = 5;
+    DSK_TRY(dev_alloc_n(m, &w.conv.mu, 5 * (size_t)D, true));
+    for (int i = 0; i < 5; ++i) DSK_TRY(W.floats_at(a.name + ".mu." + blends[i], 0, D, w.conv.mu + (size_t)i * D));
+  }
+  if (l.has_latent) {
+    const LatentSpec& a = l.latent;
+    w.dim_p = (int)up(a.dim, 32);
+    w.rot_p = (int)up(a.rot_dim, 32);
+    w.vdim_p = (int)up(a.vdim, 32);
+    w.rank_p = (int)up(a.kv_rank, 64);
+    DSK_TRY(W.floats(a.name + ".dq.norm", 0, a.q_rank, &w.l_qn));
+    DSK_TRY(W.floats(a.name + ".dkv.norm", 0, a.kv_rank, &w.l_kvn));
+    const int hd = w.dim_p + w.rot_p;
+    DSK_TRY(W.alloc(&w.l_uq, a.heads * hd, a.q_rank));
+    DSK_TRY(W.pack_heads(a.name + ".uq", a.heads, a.dim + a.rot_dim, 0, a.dim, a.q_rank, w.l_uq, 0, hd));
+    DSK_TRY(W.pack_heads(a.name + ".uq", a.heads, a.dim + a.rot_dim, a.dim, a.rot_dim, a.q_rank, w.l_uq, w.dim_p, hd));
+    DSK_TRY(W.alloc(&w.l_ukv, a.heads * (w.dim_p + w.vdim_p), a.kv_rank));
+    DSK_TRY(W.pack_heads(a.name + ".uk", a.heads, a.dim, 0, a.dim, a.kv_rank, w.l_ukv, 0, w.dim_p));
+    DSK_TRY(W.alloc(&w.l_abs, a.heads * w.rank_p, a.dim));
+    DSK_TRY(W.pack_heads(a.name + ".uk", a.heads, a.dim, 0, a.dim, a.kv_rank, w.l_abs, 0, w.rank_p, true));
+    DSK_TRY(W.pack_heads(a.name + ".uv", a.heads, a.vdim, 0, a.vdim, a.kv_rank, w.l_ukv, a.heads * w.dim_p, w.vdim_p));
+    DSK_TRY(W.matrix(a.name + ".o", D, a.heads * a.vdim, &w.l_o));
+  }
+  if (l.sandwich) {
+    DSK_TRY(W.floats(l.post, 0, D, &w.post));
+    DSK_TRY(W.floats(l.conv, D, l.taps, &w.conv.w));
+  }
+  if (l.has_dense) {
+    const DenseSpec& a = l.dense;
+    DSK_TRY(W.floats(l.ff_norm, 0, D, &w.ff_norm));
+    DSK_TRY(W.floats(l.ff_post, 0, D, &w.ff_post));
+    DSK_TRY(W.floats(l.ff_conv, D, l.taps, &w.ff_conv.w));
+    DSK_TRY(W.matrix(a.name + ".up", a.ff, D, &w.ff_up));
+    DSK_TRY(W.matrix(a.name + ".down", D, a.ff, &w.ff_down));
+    float *act = nullptr, pq[2];
+    DSK_TRY(W.floats(a.name + ".act", 0, 2, &act));
+    HIP_TRY(hipMemcpyAsync(pq, act, sizeof pq, hipMemcpyDeviceToHost, m->ctx->stream));
+    HIP_TRY(hipStreamSynchronize(m->ctx->stream));
+    auto softplus = [](double v) { return std::max(v, 0.0) + log1p(exp(-fabs(v))); };
+    w.ff_pos = (float)softplus(pq[0]);
+    w.ff_neg = (float)(0.5 + softplus(pq[1]));
   }
   if (!l.pair_a.empty()) {
     DSK_TRY(W.floats(l.pair_a, 0, D, &w.pair_a));
@@ -352,6 +469,13 @@ void layout_state(LayeredModel* m) {
       w.off_ds = take((size_t)a.heads * a.dim * a.vdim * 4);
       w.off_dc = take((size_t)2 * (a.taps - 1) * (2 * a.kv_heads * a.dim + a.heads * a.vdim) * 4);
     }
+    if (l.has_wkv) {
+      w.off_ws = take((size_t)l.wkv.heads * l.wkv.dim * l.wkv.dim * 4);
+      w.conv.off_prev = take((size_t)2 * m->s.width * 4);
+    }
+    if (l.has_latent) w.off_lc = take((size_t)l.latent.window * (w.rank_p + w.rot_p) * m->elem());
+    if (l.sandwich) w.conv.off_in = take((size_t)2 * (l.taps - 1) * m->s.width * 4);
+    if (l.has_dense) w.ff_conv.off_in = take((size_t)2 * (l.taps - 1) * m->s.width * 4);
   }
   m->seq_bytes = std::max<size_t>(off, 256);
 }
@@ -369,10 +493,15 @@ int alloc_desc(LayeredModel* m, DescBuf* d, int cap) {
   d->o_want = take(cap);
   d->o_tile = take(2 * (size_t)cap);
   d->o_chunk = take(2 * (size_t)cap);
+  d->o_single = take(cap);
   d->bytes = off;
   HIP_TRY(hipHostMalloc((void**)&d->host, off, hipHostMallocDefault));
   memset(d->host, 0, off);
   return dev_alloc(m, (void**)&d->dev, off);
+}
+
+int latent_splits(const LayeredModel* m, const LatentSpec& a) {  // workgroups for a full window
+  return (a.window + latent_keys(m->f32) - 1) / latent_keys(m->f32);
 }
 
 int alloc_work(LayeredModel* m) {
@@ -380,6 +509,8 @@ int alloc_work(LayeredModel* m) {
   const size_t n = m->piece, e = m->elem();
   const int D = s.width;
   int low = 0, out = 0, experts = 0, tmax = 1;
+  size_t hidden = 0, turn = 0, cq = 0, key = 0, kv = 0, qabs = 0, lat_part = 0, lat_ml = 0;  // (hidden: elements of a row of experts' or dense outputs)
+  bool sandwich = false;
   size_t chunk = 0, gates = 0, part = 0, arrived = 0, aq = 0, ak = 0, av = 0, dq = 0, dv = 0, dg = 0, db = 0, o = 0;
   for (size_t i = 0; i < m->L.size(); ++i) {
     const LayerSpec& l = s.layers[i];
@@ -411,10 +542,37 @@ int alloc_work(LayeredModel* m) {
       low = std::max(low, w.d_low2.rt * 16);
       out = std::max(out, w.d_o.kt * 32);
     }
+    if (l.has_wkv) {
+      const WkvSpec& a = l.wkv;
+      m->mixes = std::max(m->mixes, w.conv.n_mix);
+      chunk = std::max(chunk, a.heads * chunk_floats(a.dim));
+      o = std::max(o, (size_t)a.heads * a.dim);
+      low = std::max(low, w.w_low2.rt * 16);
+      out = std::max(out, w.w_o.kt * 32);
+    }
+    if (l.has_latent) {
+      const LatentSpec& a = l.latent;
+      m->max_window = std::max(m->max_window, a.window);
+      cq = std::max(cq, (size_t)w.l_uq.kt * 32);
+      turn = std::max(turn, (size_t)a.rot.dims);
+      m->lq_ld = std::max(m->lq_ld, w.l_uq.rt * 16 + 64);  // (the last head's columns, read in groups of 64)
+      key = std::max(key, (size_t)w.rank_p + w.rot_p);
+      kv = std::max(kv, (size_t)w.l_ukv.rt * 16);
+      qabs = std::max(qabs, (size_t)a.heads * w.rank_p);
+      lat_part = std::max(lat_part, (size_t)FEW * a.heads * latent_splits(m, a) * w.rank_p);
+      lat_ml = std::max(lat_ml, (size_t)FEW * a.heads * latent_splits(m, a) * 2);
+      out = std::max(out, w.l_o.kt * 32);
+    }
+    sandwich |= l.sandwich;
+    if (l.has_dense) {
+      m->hid_ld = std::max(m->hid_ld, w.ff_down.kt * 32);
+      hidden = std::max<size_t>(hidden, 1);
+    }
     if (l.has_moe) {
       const MoeSpec& q = l.moe;
       experts = std::max(experts, q.experts);
       tmax = std::max(tmax, q.top + (q.shared_ff > 0));
+      hidden = std::max<size_t>(hidden, q.top + (q.shared_ff > 0));
       m->hid_ld = std::max({m->hid_ld, w.e_down.kt * 32, w.e_down.shared_kt * 32});
     }
   }
@@ -425,7 +583,19 @@ int alloc_work(LayeredModel* m) {
   m->slots = tmax;
   m->ld_logits = m->head.rt * 16;
   DSK_TRY(dev_alloc_n(m, &m->x, n * D));
-  DSK_TRY(dev_alloc(m, (void**)&m->h, n * m->h_ld * e));
+  DSK_TRY(dev_alloc(m, (void**)&m->h, n * m->h_ld * e * m->mixes));
+  if (sandwich) DSK_TRY(dev_alloc_n(m, &m->h_f, n * D));
+  if (m->max_window) {
+    m->key_cap = m->piece + m->max_window;
+    DSK_TRY(dev_alloc_n(m, &m->turn, n * turn));
+    DSK_TRY(dev_alloc(m, (void**)&m->cq, n * cq * e));
+    DSK_TRY(dev_alloc(m, (void**)&m->lq, n * m->lq_ld * e));
+    DSK_TRY(dev_alloc(m, (void**)&m->lat, m->key_cap * key * e));
+    DSK_TRY(dev_alloc(m, (void**)&m->kv, m->key_cap * kv * e));
+    DSK_TRY(dev_alloc(m, (void**)&m->qabs, FEW * qabs * e));
+    DSK_TRY(dev_alloc_n(m, &m->lat_part, lat_part));
+    DSK_TRY(dev_alloc_n(m, &m->lat_ml, lat_ml));
+  }
   DSK_TRY(dev_alloc(m, (void**)&m->hw, n * m->h_ld * e));
   DSK_TRY(dev_alloc(m, (void**)&m->wide, n * m->ldw * e));
   DSK_TRY(dev_alloc_n(m, &m->narrow, n * m->ldf));
@@ -452,10 +622,10 @@ int alloc_work(LayeredModel* m) {
   }
   DSK_TRY(dev_alloc_n(m, &m->attn_part, part));
   DSK_TRY(dev_alloc_n(m, &m->attn_arrived, arrived));
+  if (hidden) DSK_TRY(dev_alloc(m, (void**)&m->hidden, n * hidden * m->hid_ld * e));
   if (experts) {
     const size_t ns = n * tmax;
     m->max_tiles = (int)(ns / MOE_TILE) + experts + 2;
-    DSK_TRY(dev_alloc(m, (void**)&m->hidden, ns * m->hid_ld * e));
     DSK_TRY(dev_alloc(m, (void**)&m->y, ns * m->y_ld * e));
     DSK_TRY(dev_alloc_n(m, &m->weight, ns));
     DSK_TRY(dev_alloc_n(m, &m->slot_pos, ns));
@@ -523,6 +693,7 @@ JoinArgs join_args(LayeredModel* m, const PassDesc& p, int l) {
   const LayerSpec& s = m->s.layers[l - 1];
   const LayerW& w = m->L[l - 1];
   j.mix_a = m->mix_a;
+  j.post_w = s.has_dense ? w.ff_post : w.post;
   if (w.pair_a) {
     j.mix_b = m->mix_b;
     j.pair_wa = w.pair_a;
@@ -638,6 +809,10 @@ DeltaArgs delta_args(LayeredModel* m, const PassDesc& p, const LayerSpec& l, con
   a.ld_low = m->low_ld;
   a.conv_w = w.d_conv;
   a.a_rate = w.d_rate;
+  a.head_decay = s.head_decay;
+  a.col_a = w.d_a;
+  a.silu_gate = s.silu_gate;
+  a.col_g = w.d_g;
   a.dt_bias = w.d_dt;
   a.out_norm = w.d_norm;
   a.q = m->dq;
@@ -653,8 +828,10 @@ DeltaArgs delta_args(LayeredModel* m, const PassDesc& p, const LayerSpec& l, con
   return a;
 }
 int delta(LayeredModel* m, const DeltaArgs& a, const LayerW& w, bool few) {
-  const LinArgs low = lin_f(w.d_low2, m->wide + (size_t)w.d_low * m->elem(), m->ldw, a.p.rows, m->low, m->low_ld);
-  DSK_TRY(run_lin(m, &low, 1, few));
+  if (!a.head_decay) {
+    const LinArgs low = lin_f(w.d_low2, m->wide + (size_t)w.d_low * m->elem(), m->ldw, a.p.rows, m->low, m->low_ld);
+    DSK_TRY(run_lin(m, &low, 1, few));
+  }
   DSK_TRY(launch_delta_prep(m->ctx->stream, a, m->f32));
   if (in_chunks(m, a.p)) DSK_TRY(launch_delta_chunks(m->ctx->stream, a, m->scan));
   else DSK_TRY(launch_delta_scan(m->ctx->stream, a));
@@ -697,13 +874,148 @@ MoeArgs moe_args(LayeredModel* m, const PassDesc& p, const LayerSpec& l, const L
   return a;
 }
 
+WkvArgs wkv_args(LayeredModel* m, const PassDesc& p, const LayerSpec& l, const LayerW& w) {
+  WkvArgs a{};
+  a.p = p;
+  a.heads = l.wkv.heads;
+  a.dim = l.wkv.dim;
+  a.eps = (float)m->s.eps;
+  a.proj_t = m->wide;
+  a.ld = m->ldw;
+  a.col_r = w.w_r;
+  a.col_k = w.w_k;
+  a.col_v = w.w_v;
+  a.col_g = w.w_g;
+  a.low_f = m->low;
+  a.ld_low = m->low_ld;
+  a.w0 = w.w_w0;
+  a.u = w.w_u;
+  a.out_norm = w.w_norm;
+  a.o = m->o;
+  a.off_s = w.off_ws;
+  a.out_t = m->out_a;
+  a.out_ld = w.w_o.kt * 32;
+  return a;
+}
+int wkv(LayeredModel* m, const WkvArgs& a, const LayerW& w, bool few) {
+  hipStream_t st = m->ctx->stream;
+  // the decay's second product multiplies 32-bit activations, in bfloat16 runs too
+  const LinArgs low = lin_f(w.w_low2, m->narrow + w.w_low, m->ldf, a.p.rows, m->low, m->low_ld);
+  DSK_TRY(few ? launch_lin_few(st, &low, 1, true) : launch_lin(st, low, true));
+  if (in_chunks(m, a.p)) DSK_TRY(launch_wkv_chunks(st, a, m->scan, m->f32));
+  else DSK_TRY(launch_wkv_scan(st, a, m->f32));
+  return launch_wkv_out(st, a, m->f32);
+}
+LatentArgs latent_args(LayeredModel* m, const PassDesc& p, const LayerSpec& l, const LayerW& w) {
+  const LatentSpec& s = l.latent;
+  LatentArgs a{};
+  a.p = p;
+  a.heads = s.heads;
+  a.dim = s.dim;
+  a.rot_dim = s.rot_dim;
+  a.vdim = s.vdim;
+  a.q_rank = s.q_rank;
+  a.kv_rank = s.kv_rank;
+  a.window = s.window;
+  a.rot_dims = s.rot.dims;
+  a.dim_p = w.dim_p;
+  a.rot_p = w.rot_p;
+  a.vdim_p = w.vdim_p;
+  a.rank_p = w.rank_p;
+  a.scale = (float)s.scale;
+  a.eps = (float)m->s.eps;
+  a.proj_f = m->narrow;
+  a.ld = m->ldf;
+  a.col_q = w.l_q;
+  a.col_kv = w.l_kv;
+  a.q_norm = w.l_qn;
+  a.kv_norm = w.l_kvn;
+  a.freq = w.freq;
+  a.cq_t = m->cq;
+  a.cq_ld = w.l_uq.kt * 32;
+  a.turn = m->turn;
+  a.q_t = m->lq;
+  a.q_ld = m->lq_ld;
+  a.lat_t = m->lat;
+  a.kv_t = m->kv;
+  a.kv_ld = w.l_ukv.rt * 16;
+  a.off_c = w.off_lc;
+  a.out_t = m->out_a;
+  a.out_ld = w.l_o.kt * 32;
+  a.splits = std::min(m->splits, latent_splits(m, s));
+  a.qa_t = m->qabs;
+  a.part = m->lat_part;
+  a.part_ml = m->lat_ml;
+  a.up_w = w.l_ukv.w;
+  a.up_kt = w.l_ukv.kt;
+  a.up_row = s.heads * w.dim_p;
+  return a;
+}
+int latent(LayeredModel* m, LatentArgs a, const LayerW& w, bool few) {
+  hipStream_t st = m->ctx->stream;
+  DSK_TRY(launch_latent_prep(st, a, m->f32));
+  auto to_t = [&](LinArgs l, void* out, int ld) {  // everything in the activations' type
+    l.n_wide = l.rt * 16;
+    l.out_t = out;
+    l.ld_t = ld;
+    return l;
+  };
+  const LinArgs uq = to_t(lin(w.l_uq, m->cq, a.cq_ld, a.p.rows), m->lq, m->lq_ld);
+  DSK_TRY(run_lin(m, &uq, 1, few));
+  if (a.p.key_rows) {
+    DSK_TRY(launch_latent_gather(st, a, m->f32));
+    const LinArgs ukv = to_t(lin(w.l_ukv, m->lat, w.rank_p + w.rot_p, a.p.key_rows), m->kv, a.kv_ld);
+    DSK_TRY(run_lin(m, &ukv, 1, false));
+    DSK_TRY(launch_latent_attn(st, a, m->f32));
+    DSK_TRY(launch_latent_store(st, a, m->f32));
+  }
+  for (a.first = 0; a.first < a.p.n_single; a.first += FEW) {
+    a.n = std::min((int)FEW, a.p.n_single - a.first);
+    LinArgs qa = to_t(lin(w.l_abs, m->lq, m->lq_ld, a.n), m->qabs, a.heads * w.rank_p);
+    qa.a_seg = w.rank_p;  // a head's features read its part of the queries
+    qa.a_ops = a.heads;
+    qa.a_stride = w.dim_p + w.rot_p;
+    if (!few) {
+      qa.row_seq = a.p.single + a.first;
+      qa.seqs = a.p.seqs;
+    }
+    DSK_TRY(launch_lin_few(st, &qa, 1, m->f32));
+    DSK_TRY(launch_latent_few(st, a, m->f32));
+  }
+  return DSK_OK;
+}
+
+ConvArgs conv_args(LayeredModel* m, const PassDesc& p, const LayerSpec& l, const ConvW& c) {
+  ConvArgs a{};
+  a.taps = l.taps;
+  a.w = c.w;
+  a.off_in = c.off_in;
+  a.mu = c.mu;
+  a.n_mix = c.n_mix;
+  a.off_prev = c.off_prev;
+  a.out_t = m->h;
+  a.ld = m->h_ld;
+  a.mix_stride = (size_t)p.rows * m->h_ld;
+  return a;
+}
+// the residual sum and norm in front of a sublayer, and the convolution a sandwich layer has there
+int enter(LayeredModel* m, JoinArgs j, const float* norm_w, const LayerSpec& s, const ConvW& c, bool few) {
+  j.norm_w = norm_w;
+  if (!s.sandwich) return launch_join(m->ctx->stream, j, m->f32);
+  const ConvArgs conv = conv_args(m, j.p, s, c);
+  if (few && m->fused_decode) {
+    j.conv = conv;
+    return launch_join(m->ctx->stream, j, m->f32);
+  }
+  j.h_f = m->h_f;
+  DSK_TRY(launch_join(m->ctx->stream, j, m->f32));
+  return launch_conv(m->ctx->stream, j.p, m->s.width, m->h_f, conv, m->f32);
+}
 int run_layer(LayeredModel* m, const PassDesc& p, int l, bool few) {
   const LayerSpec& s = m->s.layers[l];
   const LayerW& w = m->L[l];
   hipStream_t st = m->ctx->stream;
-  JoinArgs j = join_args(m, p, l);
-  j.norm_w = w.norm;
-  DSK_TRY(launch_join(st, j, m->f32));
+  DSK_TRY(enter(m, join_args(m, p, l), w.norm, s, w.conv, few));
   if (m->trace && l > 0) HIP_TRY(hipMemcpyAsync(m->trace_x + (size_t)(l - 1) * m->piece * m->s.width, m->x, (size_t)p.rows * m->s.width * 4, hipMemcpyDeviceToDevice, st));
   LinArgs pr = lin(w.proj, m->h, m->h_ld, p.rows);
   pr.n_wide = w.n_wide;
@@ -711,6 +1023,12 @@ int run_layer(LayeredModel* m, const PassDesc& p, int l, bool few) {
   pr.ld_t = m->ldw;
   pr.out_f = m->narrow;
   pr.ld_f = m->ldf;
+  if (s.has_wkv) {
+    pr.epi = LIN_TANH_F;
+    pr.a_seg = w.seg;
+    pr.a_ops = w.conv.n_mix;
+    pr.a_stride = (size_t)p.rows * m->h_ld;
+  }
   DSK_TRY(run_lin(m, &pr, 1, few));
   // the mixers' outputs and their products: attention or the only mixer in `a`, the second of a pair in `b`
   LinArgs outs[2];
@@ -729,22 +1047,32 @@ int run_layer(LayeredModel* m, const PassDesc& p, int l, bool few) {
     f.delta = delta_args(m, p, s, w);
     outs[n_out++] = lin_f(w.d_o, m->out_a, w.d_o.kt * 32, p.rows, m->mix_a, m->mix_ld);
   }
+  if (s.has_wkv) {
+    f.wkv = wkv_args(m, p, s, w);
+    outs[n_out++] = lin_f(w.w_o, m->out_a, w.w_o.kt * 32, p.rows, m->mix_a, m->mix_ld);
+  }
+  if (s.has_latent) outs[n_out++] = lin_f(w.l_o, m->out_a, w.l_o.kt * 32, p.rows, m->mix_a, m->mix_ld);
   const MoeArgs e = s.has_moe ? moe_args(m, p, s, w) : MoeArgs{};
   f.rows = p.rows;
   f.has_attn = s.has_attn;
   f.has_mlstm = s.has_mlstm;
   f.has_delta = s.has_delta;
+  f.has_wkv = s.has_wkv;
   f.has_route = s.has_moe;
   f.moe = e;
   f.splits = s.has_attn ? std::min(m->splits, (s.attn.chunk + ATTN_SPLIT_KEYS - 1) / ATTN_SPLIT_KEYS) : 0;
   f.part = m->attn_part;
   f.arrived = m->attn_arrived;
-  f.low_w = w.d_low2.w;
-  f.low_kt = w.d_low2.kt;
+  const PackedMat& low2 = s.has_wkv ? w.w_low2 : w.d_low2;
+  f.low_w = low2.w;
+  f.low_kt = low2.kt;
   f.low_a = w.low_a;
   f.low_g = w.low_g;
   f.col_low = w.d_low;
-  const bool fused = few && m->fused_decode && mix_few_fits(f);
+  f.wkv_low = m->narrow + w.w_low;
+  f.wkv_low_ld = m->ldf;
+  const bool fused = few && m->fused_decode && !s.has_latent && mix_few_fits(f);
+  if (s.has_latent) DSK_TRY(latent(m, latent_args(m, p, s, w), w, few));
   if (fused) {
     DSK_TRY(launch_mix_few(st, f, m->f32));
     m->fused_layers++;
@@ -752,6 +1080,27 @@ int run_layer(LayeredModel* m, const PassDesc& p, int l, bool few) {
     if (s.has_attn) DSK_TRY(attention(m, f.attn));
     if (s.has_mlstm) DSK_TRY(mlstm(m, f.mlstm));
     if (s.has_delta) DSK_TRY(delta(m, f.delta, w, few));
+    if (s.has_wkv) DSK_TRY(wkv(m, f.wkv, w, few));
+  }
+  if (s.has_dense) {
+    DSK_TRY(run_lin(m, outs, n_out, few));
+    JoinArgs j = join_args(m, p, l);
+    j.embed = nullptr;
+    j.y_t = nullptr;
+    j.mix_a = m->mix_a;
+    j.mix_b = nullptr;
+    j.post_w = w.post;
+    DSK_TRY(enter(m, j, w.ff_norm, s, w.ff_conv, few));
+    LinArgs u = lin(w.ff_up, m->h, m->h_ld, p.rows);
+    u.epi = LIN_XIELU;
+    u.p0 = w.ff_pos;
+    u.p1 = w.ff_neg;
+    u.n_wide = w.ff_up.rt * 16;
+    u.out_t = m->hidden;
+    u.ld_t = m->hid_ld;
+    DSK_TRY(run_lin(m, &u, 1, few));
+    const LinArgs d = lin_f(w.ff_down, m->hidden, m->hid_ld, p.rows, m->mix_a, m->mix_ld);
+    return run_lin(m, &d, 1, few);
   }
   if (!s.has_moe) return run_lin(m, outs, n_out, few);
   if (few) {
@@ -771,6 +1120,9 @@ int run_head(LayeredModel* m, int r0, int n) {
   if (m->s.softcap > 0) {
     a.epi = LIN_SOFTCAP;
     a.p0 = (float)m->s.softcap;
+  } else if (m->s.logit_scale != 1.0) {
+    a.epi = LIN_SCALE;
+    a.p0 = (float)m->s.logit_scale;
   }
   return run_lin(m, &a, 1, n <= FEW);
 }
@@ -794,6 +1146,7 @@ PassDesc pass_desc(const DescBuf& d, int rows, int n_seqs, int n_want, int n_til
   p.want = reinterpret_cast<const int*>(d.dev + d.o_want);
   p.qtile = reinterpret_cast<const int*>(d.dev + d.o_tile);
   p.chunk = reinterpret_cast<const int*>(d.dev + d.o_chunk);
+  p.single = reinterpret_cast<const int*>(d.dev + d.o_single);
   p.rows = rows;
   p.n_seqs = n_seqs;
   p.n_want = n_want;
@@ -830,6 +1183,9 @@ int run_few(LayeredModel* m, const PassDesc& p, int mode) {
   return DSK_OK;
 }
 
+// keys in front of a portion that starts at `pos` which a window of the model may reach
+int older_keys(const LayeredModel* m, int pos) { return m->max_window ? std::min(pos, m->max_window - 1) : 0; }
+
 struct Part {   // a portion of one entry inside a pass
   int entry, first, len;
 };
@@ -846,12 +1202,19 @@ int run_pass(LayeredModel* m, const dsk_step_entry* e, const std::vector<Part>& 
   DescBuf& d = few ? m->small : m->big;
   SeqDesc* sd = reinterpret_cast<SeqDesc*>(d.host);
   int *tok = reinterpret_cast<int*>(d.host + d.o_tok), *row = reinterpret_cast<int*>(d.host + d.o_row), *wn = reinterpret_cast<int*>(d.host + d.o_want),
-      *tile = reinterpret_cast<int*>(d.host + d.o_tile), *chunk = reinterpret_cast<int*>(d.host + d.o_chunk);
-  int r = 0, nt = 0, nc = 0;
+      *tile = reinterpret_cast<int*>(d.host + d.o_tile), *chunk = reinterpret_cast<int*>(d.host + d.o_chunk), *lone = reinterpret_cast<int*>(d.host + d.o_single);
+  int r = 0, nt = 0, nc = 0, ns = 0, keys = 0, max_hist = 0;
   for (size_t i = 0; i < parts.size(); ++i) {
     const Part& p = parts[i];
     Seq& q = m->seqs[e[p.entry].seq];
-    sd[i] = {q.base, r, p.len, q.pos, q.flip, nc};
+    const int hist = older_keys(m, q.pos);
+    sd[i] = {q.base, r, p.len, q.pos, q.flip, nc, keys, p.len > 1 ? hist : 0};
+    if (p.len == 1) {
+      lone[ns++] = (int)i;
+    } else {
+      keys += hist + p.len;
+      max_hist = std::max(max_hist, hist);
+    }
     for (int t = 0; t < p.len; ++t) {
       tok[r + t] = e[p.entry].tokens[p.first + t];
       row[r + t] = (int)i;
@@ -869,7 +1232,10 @@ int run_pass(LayeredModel* m, const dsk_step_entry* e, const std::vector<Part>& 
   for (size_t i = 0; i < want.size(); ++i) wn[i] = want[i];
   hipStream_t st = m->ctx->stream;
   const int nw = (int)want.size();
-  const PassDesc p = pass_desc(d, rows, (int)parts.size(), nw, nt, nc);
+  PassDesc p = pass_desc(d, rows, (int)parts.size(), nw, nt, nc);
+  p.n_single = ns;
+  p.key_rows = keys;
+  p.max_hist = max_hist;
   m->last_rows = rows;
   if (few) {
     if (mode == OUT_SAMPLE) {  // (sp_host's temperature and top_p were set by the caller)
@@ -879,6 +1245,7 @@ int run_pass(LayeredModel* m, const dsk_step_entry* e, const std::vector<Part>& 
     for (const LayerSpec& l : m->s.layers)
       for (const Part& q : parts)
         if (l.has_attn) need = std::max(need, m->seqs[e[q.entry].seq].pos % l.attn.chunk / ATTN_SPLIT_KEYS + 1);
+        else if (l.has_latent) need = std::max(need, std::min(m->seqs[e[q.entry].seq].pos, l.latent.window - 1) / latent_keys(m->f32) + 1);
     int lg = 0;
     while ((1 << lg) < need) ++lg;
     m->splits = 1 << lg;
@@ -911,6 +1278,7 @@ int run_pass(LayeredModel* m, const dsk_step_entry* e, const std::vector<Part>& 
       memcpy(next, m->next_host, (size_t)nw * 4);
     }
   } else {
+    m->splits = 1 << 30;  // (a mixer takes as many as its largest window has)
     DSK_TRY(run_body(m, d, p, false));
     const int block = mode == OUT_LOGITS ? LOGIT_ROWS : FEW;
     for (int i = 0; i < nw; i += block) {
@@ -950,7 +1318,7 @@ int run_step(LayeredModel* m, const dsk_step_entry* e, int n, int mode, float* o
   for (int i = 0; i < n; ++i) DSK_TRY(check_seq(m, e[i].seq));
   std::vector<Part> parts;
   std::vector<int> want, want_entry;
-  int rows = 0;
+  int rows = 0, keys = 0;  // keys: rows of the key workspace (latent attention)
   auto flush = [&]() -> int {
     if (parts.empty()) return DSK_OK;
     std::vector<int32_t> nx(want.size());
@@ -964,7 +1332,7 @@ int run_step(LayeredModel* m, const dsk_step_entry* e, int n, int mode, float* o
     parts.clear();
     want.clear();
     want_entry.clear();
-    rows = 0;
+    rows = keys = 0;
     return DSK_OK;
   };
   for (int i = 0; i < n; ++i) {
@@ -972,10 +1340,12 @@ int run_step(LayeredModel* m, const dsk_step_entry* e, int n, int mode, float* o
       if (e[i].want[t] <= e[i].want[t - 1]) DSK_FAIL(DSK_ERR_UNSUPPORTED, "step: the wanted places must ascend");
     for (int done = 0; done < e[i].n_tokens;) {
       const int len = std::min(e[i].n_tokens - done, m->piece - rows);
-      if (len == 0) {
+      const int k = m->max_window && len > 1 ? older_keys(m, m->seqs[e[i].seq].pos) + len : 0;
+      if (len == 0 || (rows && keys + k > m->key_cap && k)) {  // (behind a flush everything fits)
         DSK_TRY(flush());
         continue;
       }
+      keys += k;
       parts.push_back({i, done, len});
       if (mode == OUT_LOGITS) {
         for (int w = 0; w < e[i].n_want; ++w)
@@ -1162,6 +1532,11 @@ double l_active_bytes(const dsk_model* h, int pos) {
       b += 2.0 * (double)w.a_o.elems() + (double)(pos % l.attn.chunk) * l.attn.kv_heads * (l.attn.dim + l.attn.vdim) * m->elem();
     if (l.has_mlstm) b += 2.0 * (double)w.m_o.elems() + 8.0 * l.mlstm.heads * l.mlstm.dim * (l.mlstm.vdim + 1);
     if (l.has_delta) b += 2.0 * (double)(w.d_o.elems() + w.d_low2.elems()) + 8.0 * l.delta.heads * l.delta.dim * l.delta.vdim;
+    if (l.has_wkv) b += 2.0 * (double)(w.w_o.elems() + w.w_low2.elems()) + 8.0 * l.wkv.heads * l.wkv.dim * l.wkv.dim;
+    if (l.has_latent)
+      b += 2.0 * (double)(w.l_uq.elems() + w.l_abs.elems() + (size_t)l.latent.heads * w.vdim_p * w.rank_p + w.l_o.elems()) +
+           (double)std::min(pos + 1, l.latent.window) * (w.rank_p + w.rot_p) * m->elem();
+    if (l.has_dense) b += 2.0 * (double)(w.ff_up.elems() + w.ff_down.elems());
     if (l.has_moe) {
       b += 2.0 * l.moe.top * (double)(w.e_up.stride + w.e_down.stride);
       if (l.moe.shared_ff) b += 1024.0 * ((double)w.e_up.shared_kt * w.e_up.shared_rt + (double)w.e_down.shared_kt * w.e_down.shared_rt);

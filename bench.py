@@ -71,7 +71,8 @@ def parse():
     ap.add_argument("--cpu-seconds", type=float, default=12.0)
     ap.add_argument("--profile-steps", type=int, default=4)
     ap.add_argument("--layered", default="", choices=["", "lite", "wide"],
-                    help="instead of the default workload: prefill / decode throughput of the layered design (Timerax) at real layer sizes")
+                    help="instead of the default workload: prefill / decode throughput of a layered design at real layer sizes")
+    ap.add_argument("--layered-design", default="timerax", choices=["timerax", "ranutar"])
     return ap.parse_args()
 
 
@@ -224,7 +225,7 @@ def main():
     a = parse()
     if a.layered:
         from tools import layered_bench
-        print(json.dumps(layered_bench.measure(a.layered)), flush=True)
+        print(json.dumps(layered_bench.measure(a.layered, design=a.layered_design)), flush=True)
         return
     rank = int(os.environ.get("RANK", "0"))
     local_rank = int(os.environ.get("LOCAL_RANK", "0"))

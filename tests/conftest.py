@@ -57,3 +57,17 @@ def ctx():
     c = dsk.Ctx(0)
     yield c
     c.close()
+
+
+@pytest.fixture
+def case(ctx, tmp_path):
+    """layered_util.Case of a configuration, closed behind the test"""
+    from tests import layered_util as U
+    made = []
+
+    def make(c, **kw):
+        made.append(U.Case(ctx, tmp_path / str(len(made)), c, **kw))
+        return made[-1]
+    yield make
+    for m in made:
+        m.lm.close()

@@ -1,4 +1,5 @@
-"""Layered designs on the GPU against their plain statement (oracle/layered.py), through the library's own entry points.
+"""Layered designs on the GPU against their plain statement (oracle/layered.py), through the library's own entry points: Timerax's mechanisms
+one by one (Ranutar's are in test_ranutar_gpu.py), then both whole designs.
 
 32-bit runs are held to 1e-5 of the residual stream's (or the logits') scale, bfloat16 runs to a few percent.  The models are tiny,
 have random weights and sizes that no other file uses; attention scales are large enough for single keys to dominate, so that a key
@@ -16,48 +17,13 @@ from tests import layered_util as U
 
 pytestmark = pytest.mark.gpu
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
-F32, B16 = 1e-5, 0.06
+F32, B16 = U.F32, U.B16
 
 
-class Case:
-    """one model on both sides"""
-
-    def __init__(self, ctx, tmp, c, seed=0, dtype="float32", options=None, edit=None):
-        import dsk
-        self.c, self.W = c, U.weights(c, seed)
-        if edit:
-            edit(self.W)
-            self.W = {k: U.bf16(v) for k, v in self.W.items()}
-        self.dir = U.save(tmp, c, self.W)
-        self.lm = dsk.LM(ctx, self.dir, dtype, options)
-        self.ref = O.Model(c, self.W)
-        self.tol = F32 if dtype == "float32" else B16
-
-    def tokens(self, n, seed=1):
-        return np.random.default_rng(seed).integers(0, self.c["vocab"], n)
-
-    def want(self, tokens):
-        return self.ref.run(O.Sequence(self.ref), tokens)
-
-    def got(self, tokens, cuts=()):
-        """logits of one sequence run in portions"""
-        s = self.lm.seq_open()
-        out = [self.lm.step([(s, p, range(len(p)))]) for p in np.split(np.asarray(tokens), list(cuts)) if len(p)]
-        assert self.lm.seq_pos(s) == len(tokens)
-        self.lm.seq_close(s)
-        return np.concatenate(out)
-
-
-@pytest.fixture
-def case(ctx, tmp_path):
-    made = []
-
-    def make(c, **kw):
-        made.append(Case(ctx, tmp_path / str(len(made)), c, **kw))
-        return made[-1]
-    yield make
-    for m in made:
-        m.lm.close()
+@pytest.fixture(params=[U.mixed, U.sandwich_mixed], ids=["Timerax", "Ranutar"])
+def design(request):
+    """a configuration with every mechanism of a design"""
+    return request.param
 
 
 def only_left(W):   # the recurrent half of every pair silenced
@@ -79,20 +45,7 @@ def no_mixers(W):
 
 
 def check_trace(K, n, tol=None, cuts=()):
-    """residual stream behind every layer, prompt in one step; then logits, also cut"""
-    t = K.tokens(n)
-    trace = []
-    want = K.ref.run(O.Sequence(K.ref), t, trace)
-    K.lm.set_trace(True)
-    s = K.lm.seq_open()
-    got = K.lm.step([(s, t, range(n))])
-    for l in range(len(K.c["layers"])):
-        assert U.err(K.lm.trace_rows(l, n), trace[l]) < (tol or K.tol), l
-    K.lm.seq_close(s)
-    K.lm.set_trace(False)
-    assert U.err(got, want) < (tol or K.tol)
-    for cut in cuts:
-        assert U.err(K.got(t, cut), want) < (tol or K.tol), cut
+    K.check_trace(n, tol, cuts)
 
 
 # ---- each mechanism alone ------------------------------------------------------------------------------------
@@ -163,12 +116,12 @@ def test_logits_without_and_with_a_soft_cap(case):
 
 # ---- the whole design ------------------------------------------------------------------------------------------
 @pytest.mark.parametrize("width", [120, 64, 77, 300], ids=lambda w: f"width-{w}")
-def test_all_layers_in_32_bit(case, width):
-    check_trace(case(U.mixed(width), seed=width), 100, tol=2e-5, cuts=([64], [2, 4, 6, 8], [19, 38, 57]))
+def test_all_layers_in_32_bit(design, case, width):
+    check_trace(case(design(width), seed=width), 100, tol=2e-5, cuts=([64], [2, 4, 6, 8], [19, 38, 57]))
 
 
-def test_bfloat16_stays_close(case):
-    K = case(U.mixed(), dtype="bfloat16")
+def test_bfloat16_stays_close(design, case):
+    K = case(design(), dtype="bfloat16")
     t = K.tokens(100)
     want = K.want(t)
     for got in (K.got(t), K.got(t, range(40, 100))):
@@ -176,22 +129,22 @@ def test_bfloat16_stays_close(case):
 
 
 @pytest.mark.parametrize("size", [2, 3, 7, 16, 17, 33, 64])
-def test_portions_of_a_prompt(case, size):
-    K = case(U.mixed())
+def test_portions_of_a_prompt(design, case, size):
+    K = case(design())
     t = K.tokens(130)
     assert U.err(K.got(t, range(size, 130, size)), K.want(t)) < 2e-5
 
 
-def test_portions_larger_than_one_pass(case):
-    K = case(U.mixed(), options="piece_tokens=48")
+def test_portions_larger_than_one_pass(design, case):
+    K = case(design(), options="piece_tokens=48")
     t = K.tokens(131)
     assert U.err(K.got(t), K.want(t)) < 2e-5
     assert U.err(K.got(t, [100]), K.want(t)) < 2e-5
 
 
 @pytest.mark.parametrize("options", ["fused_decode=0", "decode_graph=0", "chunk_scan=0", "fused_decode=0,decode_graph=0,chunk_scan=0"])
-def test_every_option_computes_the_same(case, options):
-    K, L = case(U.mixed()), case(U.mixed(), options=options)
+def test_every_option_computes_the_same(design, case, options):
+    K, L = case(design()), case(design(), options=options)
     t = K.tokens(70)
     a, b = K.got(t, range(40, 70)), L.got(t, range(40, 70))
     assert U.err(a, b) < 2e-5
@@ -200,8 +153,8 @@ def test_every_option_computes_the_same(case, options):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-def test_unequal_requests_together_and_alone(case, dtype):
-    K = case(U.mixed(), dtype=dtype)
+def test_unequal_requests_together_and_alone(design, case, dtype):
+    K = case(design(), dtype=dtype)
     lens = [1, 37, 64, 5, 20]
     toks = [K.tokens(n + 25, seed=n) for n in lens]
     seqs = [K.lm.seq_open() for _ in lens]
@@ -222,8 +175,8 @@ def test_unequal_requests_together_and_alone(case, dtype):
         assert U.err(np.array(got[j]), alone, part) < tol
 
 
-def test_more_sequences_than_one_decode_launch_takes(case):
-    K = case(U.mixed())
+def test_more_sequences_than_one_decode_launch_takes(design, case):
+    K = case(design())
     toks = [K.tokens(12, seed=n) for n in range(21)]
     seqs = [K.lm.seq_open() for _ in toks]
     K.lm.step([(s, t[:8], []) for s, t in zip(seqs, toks)])
@@ -233,8 +186,8 @@ def test_more_sequences_than_one_decode_launch_takes(case):
         assert U.err(row[None], K.want(t)[-1:]) < 2e-5
 
 
-def test_slots_are_used_again_without_a_trace_of_what_they_held(case):
-    K = case(U.mixed())
+def test_slots_are_used_again_without_a_trace_of_what_they_held(design, case):
+    K = case(design())
     t = K.tokens(50, seed=5)
     fresh = K.got(t, range(30, 50))
     seqs = [K.lm.seq_open() for _ in range(6)]
@@ -280,15 +233,15 @@ def test_attention_parts_meet_in_decoding(case):
     assert K.lm.info("graph_captured") >= 3
 
 
-def test_long_decoding(case):
-    K = case(U.mixed())
+def test_long_decoding(design, case):
+    K = case(design())
     t = K.tokens(260)
     assert U.err(K.got(t, range(3, 260)), K.want(t)) < 3e-5
     assert K.lm.info("graph_steps") > 200
 
 
-def test_first_tokens(case):
-    K = case(U.mixed())
+def test_first_tokens(design, case):
+    K = case(design())
     t = K.tokens(6)
     want = K.want(t)
     for cuts in ([], [1], [1, 2], [1, 2, 3, 4, 5], [2, 3]):
@@ -296,9 +249,9 @@ def test_first_tokens(case):
 
 
 # ---- entry points ----------------------------------------------------------------------------------------------------
-def test_single_sequence_calls(case):
+def test_single_sequence_calls(design, case):
     import dsk
-    K = case(U.mixed())
+    K = case(design())
     t = K.tokens(30)
     want = K.want(t)
     assert U.err(K.lm.hydrate(t[:20], 0, dsk.MODE_OUTPUT_LOGITS)[None], want[19:20]) < 2e-5
@@ -312,8 +265,8 @@ def test_single_sequence_calls(case):
     assert U.err(K.lm.forward(int(t[0]), 0)[None], want[:1]) < 2e-5   # position 0 starts anew
 
 
-def test_sampling_follows_the_sampler(case, ctx):
-    K = case(U.mixed())
+def test_sampling_follows_the_sampler(design, case, ctx):
+    K = case(design())
     t = K.tokens(15)
     coins = np.linspace(0.02, 0.98, 7).astype(np.float32)
     for temperature, top_p in ((0.0, 1.0), (1.0, 1.0), (2.5, 0.9)):
@@ -329,8 +282,8 @@ def test_sampling_follows_the_sampler(case, ctx):
             K.lm.seq_close(s)
 
 
-def test_greedy_generation(case):
-    K = case(U.mixed())
+def test_greedy_generation(design, case):
+    K = case(design())
     prompts = [K.tokens(n, seed=n) for n in (1, 9, 30, 4, 17)]
     news = [12, 20, 7, 1, 16]
     for max_batch in (16, 2):
@@ -371,8 +324,8 @@ def test_bad_weights_and_steps_are_errors(case, ctx, tmp_path):
     assert K.lm.seq_pos(s) == 0
 
 
-def test_trace_runner(case, tmp_path):
-    K = case(U.mixed())
+def test_trace_runner(design, case, tmp_path):
+    K = case(design())
     a, b = K.tokens(12, 1), K.tokens(9, 2)
     steps = [{"step": 0, "entries": [{"id": "x", "tokens": a[:10].tolist(), "want": [9, 0]}, {"id": "y", "tokens": b[:7].tolist(), "want": []}], "end": []},
              {"step": 1, "entries": [{"id": "x", "tokens": a[10:11].tolist(), "want": []}, {"id": "y", "tokens": b[7:8].tolist(), "want": []}], "end": []},
@@ -393,8 +346,8 @@ def test_trace_runner(case, tmp_path):
     assert U.err(read(2), np.array([wa[11], wb[8]])) < 2e-5 and U.err(read(3), wb[2:3]) < 2e-5
 
 
-def test_generate_command(case):
-    K = case(U.mixed())
+def test_generate_command(design, case):
+    K = case(design())
     prompts = [K.tokens(5, 1).tolist(), K.tokens(11, 2).tolist()]
     r = subprocess.run([os.path.join(ROOT, "bin", "generate"), "--model", K.dir, "--dtype", "float32", "-n", "6"] + [",".join(map(str, p)) for p in prompts],
                        capture_output=True, timeout=110)

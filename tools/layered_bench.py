@@ -1,11 +1,12 @@
-"""Prompt and decode throughput of a layered design (Timerax) at sizes that resemble a real model's layers, random weights, beside the
-DeepSeek engine's model of the same width, depth and expert sizes.
+"""Prompt and decode throughput of a layered design at sizes that resemble a real model's layers, random weights, beside the closest other
+model of the same width and depth: Timerax beside the DeepSeek engine's model of the same expert sizes, Ranutar beside Timerax.
 
-  python bench.py --layered lite            (this module's measure(), one JSON line)
+  python bench.py --layered lite [--layered-design ranutar]           (this module's measure(), one JSON line)
   python tools/layered_bench.py --size wide --prompt 2048 --batch 1,16 --no-compare
 
   lite   27 layers of width 2048, 64 experts top 6 of 1408, shared expert 2816     (DeepSeek-V2-Lite's shapes; FP16 weights there)
   wide    3 layers of width 7168, 256 experts top 8 of 2048, shared expert 2048    (DeepSeek-V3's shapes; Q2_K weights there)
+Ranutar's dense feed-forwards have as many weights as Timerax reads per token.
 """
 import argparse
 import json
@@ -36,6 +37,22 @@ def config(size: str) -> dict:
             "layers": [delta, delta, par] * (1 if wide else 9)}
 
 
+def ranutar(size: str) -> dict:
+    wide = size == "wide"
+    D, heads = (7168, 64) if wide else (2048, 16)
+    mlp = {"kind": "dense", "ff": 27648 if wide else 16896}
+    wkv = {"type": "wkv", "mixer": {"heads": D // 64, "dim": 64}, "mlp": mlp}
+    delta = {"type": "delta", "mixer": {"conv": 4, "dim": 128, "heads": heads, "kv_heads": heads, "vdim": 128}, "mlp": mlp}
+    lat = {"type": "latent_attention", "mlp": mlp, "mixer": {
+        "heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": 1536, "kv_rank": 512, "mask": {"size": 4096}, "scale": 0.0721688,
+        "rot": {"base": 500000.0, "dims": 64}}}
+    return {"architecture": "Ranutar", "width": D, "vocab": 129280 if wide else 102400, "norm": {"eps": 1e-6}, "canon": {"taps": 4}, "logit_scale": 0.5,
+            "layers": [wkv, delta, lat] * (1 if wide else 9)}
+
+
+CONFIGS = {"timerax": config, "ranutar": ranutar}
+
+
 def timed(fn, reps):
     best = 1e9
     for _ in range(reps):
@@ -45,9 +62,9 @@ def timed(fn, reps):
     return best
 
 
-def layered(ctx, size, prompts, batches, steps=32, ctx_len=512, reps=2, graph=True):
+def layered(ctx, size, prompts, batches, steps=32, ctx_len=512, reps=2, graph=True, design="timerax"):
     import dsk
-    c = config(size)
+    c = CONFIGS[design](size)
     M = dsk.LM(ctx, dtype="bfloat16", config=c, seed=1, options=f"piece_tokens={max(2048, min(8192, max(prompts)))},decode_graph={int(graph)}")
     rng = np.random.default_rng(0)
     toks = rng.integers(0, c["vocab"], max(prompts + [ctx_len]) + 1)
@@ -116,16 +133,18 @@ def deepseek(ctx, size, prompts, steps=32, ctx_len=512, reps=2, graph=True):
     return out
 
 
-def measure(size="lite", prompts=(512, 2048), batches=(1, 4, 16), compare=True, steps=32, graph=True, ours=True):
+def measure(size="lite", prompts=(512, 2048), batches=(1, 4, 16), compare=True, steps=32, graph=True, ours=True, design="timerax"):
     import dsk
     ctx = dsk.Ctx(0)
-    out = {"metric": f"layered design (Timerax) prefill and decode throughput, {size}", "unit": "tok/s", "data": "synthetic (random weights)",
+    out = {"metric": f"layered design ({design.capitalize()}) prefill and decode throughput, {size}", "unit": "tok/s", "data": "synthetic (random weights)",
            "dtype": "bf16"}
     if ours:
-        out["timerax"] = layered(ctx, size, list(prompts), list(batches), steps, graph=graph)
-        out["value"] = out["timerax"]["decode"][str(batches[0])]["tok_s"]
-    if compare:
+        out[design] = layered(ctx, size, list(prompts), list(batches), steps, graph=graph, design=design)
+        out["value"] = out[design]["decode"][str(batches[0])]["tok_s"]
+    if compare and design == "timerax":
         out["deepseek"] = deepseek(ctx, size, [p for p in prompts if p <= 2048], steps, graph=graph)
+    elif compare:
+        out["timerax"] = layered(ctx, size, list(prompts), list(batches), steps, graph=graph)
     ctx.close()
     return out
 
@@ -133,15 +152,16 @@ def measure(size="lite", prompts=(512, 2048), batches=(1, 4, 16), compare=True, 
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--size", default="lite", choices=["lite", "wide"])
+    ap.add_argument("--design", default="timerax", choices=sorted(CONFIGS))
     ap.add_argument("--prompt", default="512,2048")
     ap.add_argument("--batch", default="1,4,16")
     ap.add_argument("--steps", type=int, default=32)
     ap.add_argument("--no-compare", action="store_true")
-    ap.add_argument("--only-compare", action="store_true", help="the DeepSeek model alone")
+    ap.add_argument("--only-compare", action="store_true", help="the model it is compared with alone")
     ap.add_argument("--no-graph", action="store_true", help="decode steps launched one by one (kernel traces)")
     a = ap.parse_args()
     print(json.dumps(measure(a.size, [int(v) for v in a.prompt.split(",")], [int(v) for v in a.batch.split(",")], not a.no_compare, a.steps,
-                             not a.no_graph, not a.only_compare)))
+                             not a.no_graph, not a.only_compare, a.design)))
 
 
 if __name__ == "__main__":

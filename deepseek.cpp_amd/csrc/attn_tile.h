@@ -1,6 +1,6 @@
 // attn_tile.h -- softmax attention of 64 queries of one head over a contiguous range of keys, for the attention kernels of layered models.
 //
-// 4 waves of 16 queries, key tiles of 32 through LDS, online softmax in 32-bit.  Scores come out of the MFMA with the query in the lane
+// 4 waves of 16 queries, key tiles of 64 through LDS, online softmax in 32-bit.  Scores come out of the MFMA with the query in the lane
 // and four keys in the registers, which is the operand order of the second product when v's key order is permuted alike: the weights
 // never leave their registers.  The next tile's keys and values travel to registers while the current one is worked off.
 #pragma once
@@ -9,16 +9,17 @@
 
 #include <math.h>
 
-// LDS: a tile of 32 keys as fragments [2 x 16 keys][dim / 32][64 lanes][8], then v transposed [vdim][32 keys + pad]
+// LDS: a tile of 64 keys as fragments [4 x 16 keys][dim / 32][64 lanes][8], then v transposed [vdim][64 keys + pad]
+enum { ATTN_KEYS = 64 };
 template <typename T>
 struct VT {
-  enum { LD = sizeof(T) == 2 ? 40 : 36 };  // elements per row of the transposed v tile
+  enum { LD = ATTN_KEYS + (sizeof(T) == 2 ? 8 : 4) };  // elements per row of the transposed v tile
 };
 template <typename T>
 static size_t attn_tile_lds(int dim_p, int vdim_p) {
-  return ((size_t)32 * dim_p + (size_t)vdim_p * VT<T>::LD) * sizeof(T);
+  return ((size_t)ATTN_KEYS * dim_p + (size_t)vdim_p * VT<T>::LD) * sizeof(T);
 }
-// weights x values for the 32 keys of a tile: keys 4 g + i of the first 16 and of the second 16 (g = lane / 16)
+// weights x values for 32 keys of a tile: keys 4 g + i of the first 16 and of the second 16 (g = lane / 16)
 DEV f32x4 mma_pv(const bf16* v, const f32x4& p0, const f32x4& p1, const f32x4& acc) {
   typedef bf16 b4 __attribute__((ext_vector_type(4)));
   const b4 v0 = *reinterpret_cast<const b4*>(v), v1 = *reinterpret_cast<const b4*>(v + 16);
@@ -42,11 +43,11 @@ DEV void attn_tile(const Keys& src, const SeqDesc& sq, int q0, int kts, int vts,
   typedef typename Frag<T>::type frag;
   typedef typename Frag<T>::four four;
   extern __shared__ __attribute__((aligned(16))) char lds[];
-  constexpr int KI = KT / 2, VI = (VTL + 7) / 8;         // what a thread loads of a tile: KI key groups, VI times 4 keys x 4 channels
+  constexpr int NS = ATTN_KEYS / 16, KI = KT * NS / 4, VI = (VTL * NS + 15) / 16;  // a thread's share of a tile: KI key groups, VI times 4 keys x 4 channels
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int nq = min(64, sq.len - q0);
   T* kf = reinterpret_cast<T*>(lds);                     // fragments of the key tile
-  T* vt = kf + (size_t)2 * kts * 512;                    // transposed values
+  T* vt = kf + (size_t)NS * kts * 512;                   // transposed values
   const int my_q = min(q0 + wave * 16 + (lane & 15), sq.len - 1);
   const int my_pos = sq.pos0 + my_q, my_first = src.first(my_pos);
   frag q[KT];
@@ -65,37 +66,37 @@ DEV void attn_tile(const Keys& src, const SeqDesc& sq, int q0, int kts, int vts,
 #pragma unroll
     for (int u = 0; u < KI; ++u) {
       const int i = tid + 256 * u;
-      if (i < 32 * ng) rk[u] = src.k(min(j0 + i / ng, last), i % ng);
+      if (i < ATTN_KEYS * ng) rk[u] = src.k(min(j0 + i / ng, last), i % ng);
     }
 #pragma unroll
     for (int u = 0; u < VI; ++u) {
       const int i = tid + 256 * u;
-      if (i < 8 * nv)
+      if (i < ATTN_KEYS / 4 * nv)
 #pragma unroll
         for (int k = 0; k < 4; ++k) rv[u][k] = src.v(min(j0 + i / nv * 4 + k, last), i % nv * 4);
     }
   };
   fetch(first);
-  for (int j0 = first; j0 <= last; j0 += 32) {
+  for (int j0 = first; j0 <= last; j0 += ATTN_KEYS) {
     __syncthreads();
 #pragma unroll
     for (int u = 0; u < KI; ++u) {
       const int i = tid + 256 * u, key = i / ng, gr = i % ng;
-      if (i < 32 * ng) *reinterpret_cast<frag*>(kf + (((size_t)(key >> 4) * kts + (gr >> 2)) * 64 + (gr & 3) * 16 + (key & 15)) * 8) = rk[u];
+      if (i < ATTN_KEYS * ng) *reinterpret_cast<frag*>(kf + (((size_t)(key >> 4) * kts + (gr >> 2)) * 64 + (gr & 3) * 16 + (key & 15)) * 8) = rk[u];
     }
 #pragma unroll
     for (int u = 0; u < VI; ++u) {
       const int i = tid + 256 * u, kq = i / nv, c = i % nv * 4;
-      if (i < 8 * nv)
+      if (i < ATTN_KEYS / 4 * nv)
 #pragma unroll
         for (int e = 0; e < 4; ++e) *reinterpret_cast<four*>(vt + (size_t)(c + e) * VT<T>::LD + kq * 4) = four{rv[u][0][e], rv[u][1][e], rv[u][2][e], rv[u][3][e]};
     }
     __syncthreads();
-    if (j0 + 32 <= last) fetch(j0 + 32);
+    if (j0 + ATTN_KEYS <= last) fetch(j0 + ATTN_KEYS);
     if (wave * 16 >= nq || j0 > sq.pos0 + q0 + min(wave * 16 + 15, nq - 1)) continue;  // (barriers above: every wave passes them)
-    f32x4 s[2];
+    f32x4 s[NS];
 #pragma unroll
-    for (int t = 0; t < 2; ++t) {
+    for (int t = 0; t < NS; ++t) {
       s[t] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int kt = 0; kt < KT; ++kt)
@@ -103,7 +104,7 @@ DEV void attn_tile(const Keys& src, const SeqDesc& sq, int q0, int kts, int vts,
     }
     float mx = m;
 #pragma unroll
-    for (int t = 0; t < 2; ++t)
+    for (int t = 0; t < NS; ++t)
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int pos = j0 + t * 16 + (lane >> 4) * 4 + i;
@@ -116,7 +117,7 @@ DEV void attn_tile(const Keys& src, const SeqDesc& sq, int q0, int kts, int vts,
     const float old = expf(m - ref);
     float sum = 0.f;
 #pragma unroll
-    for (int t = 0; t < 2; ++t)
+    for (int t = 0; t < NS; ++t)
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         s[t][i] = expf(s[t][i] - ref);
@@ -130,7 +131,8 @@ DEV void attn_tile(const Keys& src, const SeqDesc& sq, int q0, int kts, int vts,
     for (int i = 0; i < VTL; ++i)
       if (i < vts) {
         o[i] *= old;
-        o[i] = mma_pv(vt + (size_t)(i * 16 + (lane & 15)) * VT<T>::LD + (lane >> 4) * 4, s[0], s[1], o[i]);
+#pragma unroll
+        for (int t = 0; t < NS; t += 2) o[i] = mma_pv(vt + (size_t)(i * 16 + (lane & 15)) * VT<T>::LD + t * 16 + (lane >> 4) * 4, s[t], s[t + 1], o[i]);
       }
   }
   const int qi = wave * 16 + (lane & 15);

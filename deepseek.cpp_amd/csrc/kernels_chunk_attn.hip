@@ -84,9 +84,9 @@ struct ChunkKeys {
 };
 template <typename T, int KT, int VTL>
 __global__ __launch_bounds__(256) void chunk_attn_kernel(const ChunkAttnArgs a) {
-  const int h = blockIdx.y;
-  const SeqDesc s = a.p.seqs[a.p.qtile[2 * blockIdx.x]];
-  attn_tile<T, KT, VTL>(ChunkKeys<T>{a, s, h, h / (a.heads / a.kv_heads)}, s, a.p.qtile[2 * blockIdx.x + 1], a.dim_p >> 5, a.vdim_p >> 4, a.vdim, a.scale,
+  const int h = blockIdx.y, tile = gridDim.x - 1 - blockIdx.x;  // (a sequence's last tiles have the most keys: they start first)
+  const SeqDesc s = a.p.seqs[a.p.qtile[2 * tile]];
+  attn_tile<T, KT, VTL>(ChunkKeys<T>{a, s, h, h / (a.heads / a.kv_heads)}, s, a.p.qtile[2 * tile + 1], a.dim_p >> 5, a.vdim_p >> 4, a.vdim, a.scale,
                         reinterpret_cast<T*>(a.out_t) + h * a.vdim, a.out_ld);
 }
 

@@ -28,52 +28,104 @@ DEV void store_v(S* p, const float (&v)[V]) {
     p[0] = (S)v[0];
   }
 }
-// y, or its blends with the previous token's y, of V channels from c on
-template <typename T, int V>
-DEV void store_blends(const ConvArgs& a, int D, int row, int c, const float (&y)[V], const float (&prev)[V]) {
-  T* out = reinterpret_cast<T*>(a.out_t) + (size_t)row * a.ld + c;
-  if (!a.mu) {
-    store_v<T, V>(out, y);
-    return;
-  }
-  for (int s = 0; s < a.n_mix; ++s) {
-    float m[V];
-    load_v<float, V>(a.mu + (size_t)s * D + c, true, m);
-#pragma unroll
-    for (int e = 0; e < V; ++e) m[e] = y[e] + (prev[e] - y[e]) * m[e];
-    store_v<T, V>(out + s * a.mix_stride, m);
-  }
-}
-// a sequence's only token of the pass: V channels of h through the convolution; keeps the inputs (and y) for the next token
-template <typename T, int V>
-DEV void conv_one(const JoinArgs& j, int row, int c, const float (&h)[V]) {
-  const ConvArgs& a = j.conv;
-  const SeqDesc s = j.p.seqs[j.p.row_seq[row]];
-  const int D = j.width, taps = a.taps;
-  const float* hist = reinterpret_cast<const float*>(s.state + a.off_in) + (size_t)s.flip * (taps - 1) * D + c;
-  float* next = reinterpret_cast<float*>(s.state + a.off_in) + (size_t)(s.flip ^ 1) * (taps - 1) * D + c;
-  float y[V], prev[V];
-#pragma unroll
-  for (int e = 0; e < V; ++e) y[e] = 0.f;
-#pragma unroll 4
-  for (int t = 0; t < taps - 1; ++t) {
-    float old[V];
-    load_v<float, V>(hist + (size_t)t * D, s.pos0 - (taps - 1) + t >= 0, old);
-#pragma unroll
-    for (int e = 0; e < V; ++e) y[e] += old[e] * a.w[(size_t)(c + e) * taps + t];
-    if (t > 0) store_v<float, V>(next + (size_t)(t - 1) * D, old);
-  }
-  if (taps > 1) store_v<float, V>(next + (size_t)(taps - 2) * D, h);
-#pragma unroll
-  for (int e = 0; e < V; ++e) y[e] = h[e] + (y[e] + h[e] * a.w[(size_t)(c + e) * taps + taps - 1]);
-  if (a.mu) {
+// A sequence's only token of the pass: V channels of h through the convolution.  What that needs from memory is requested at once (up to
+// MAX_TAPS taps and MAX_MIX blends; more go one after the other), early enough to be there when h is.
+template <int V>
+struct ConvOne {
+  enum { MAX_TAPS = 4, MAX_MIX = 5 };
+  float old[MAX_TAPS - 1][V], w[V][MAX_TAPS], mu[MAX_MIX][V], prev[V];
+  const float* hist;
+  float *next, *p_next;
+  bool small;
+  DEV void load(const JoinArgs& j, const SeqDesc& s, int c) {
+    const ConvArgs& a = j.conv;
+    const int D = j.width, taps = a.taps;
+    const bool in = c < D;
+    small = taps <= MAX_TAPS && a.n_mix <= MAX_MIX;
+    hist = reinterpret_cast<const float*>(s.state + a.off_in) + (size_t)s.flip * (taps - 1) * D + c;
+    next = reinterpret_cast<float*>(s.state + a.off_in) + (size_t)(s.flip ^ 1) * (taps - 1) * D + c;
     float* P = reinterpret_cast<float*>(s.state + a.off_prev) + c;
-    load_v<float, V>(P + (size_t)s.flip * D, s.pos0 > 0, prev);
-    store_v<float, V>(P + (size_t)(s.flip ^ 1) * D, y);
+    p_next = P + (size_t)(s.flip ^ 1) * D;
+    load_v<float, V>(P + (size_t)s.flip * D, in && a.mu && s.pos0 > 0, prev);
+    if (!small || !in) return;
+#pragma unroll
+    for (int t = 0; t < MAX_TAPS - 1; ++t) load_v<float, V>(hist + (size_t)t * D, t < taps - 1 && s.pos0 - (taps - 1) + t >= 0, old[t]);
+#pragma unroll
+    for (int e = 0; e < V; ++e)
+#pragma unroll
+      for (int t = 0; t < MAX_TAPS; ++t) w[e][t] = t < taps ? a.w[(size_t)(c + e) * taps + t] : 0.f;
+#pragma unroll
+    for (int i = 0; i < MAX_MIX; ++i) load_v<float, V>(a.mu + (size_t)i * D + c, a.mu && i < a.n_mix, mu[i]);
   }
-  store_blends<T, V>(a, D, row, c, y, prev);
+  template <typename T>
+  DEV void run(const JoinArgs& j, int row, int pos0, int c, const float (&h)[V]) {
+    const ConvArgs& a = j.conv;
+    const int D = j.width, taps = a.taps;
+    T* out = reinterpret_cast<T*>(a.out_t) + (size_t)row * a.ld + c;
+    float y[V];
+#pragma unroll
+    for (int e = 0; e < V; ++e) y[e] = 0.f;
+    if (small) {
+#pragma unroll
+      for (int t = 0; t < MAX_TAPS; ++t)
+#pragma unroll
+        for (int e = 0; e < V; ++e) y[e] += t < taps ? (t == taps - 1 ? h[e] : old[t < MAX_TAPS - 1 ? t : 0][e]) * w[e][t] : 0.f;
+#pragma unroll
+      for (int t = 1; t < MAX_TAPS - 1; ++t)
+        if (t < taps - 1) store_v<float, V>(next + (size_t)(t - 1) * D, old[t]);
+    } else {
+      for (int t = 0; t < taps - 1; ++t) {
+        float o[V];
+        load_v<float, V>(hist + (size_t)t * D, pos0 - (taps - 1) + t >= 0, o);
+#pragma unroll
+        for (int e = 0; e < V; ++e) y[e] += o[e] * a.w[(size_t)(c + e) * taps + t];
+        if (t > 0) store_v<float, V>(next + (size_t)(t - 1) * D, o);
+      }
+#pragma unroll
+      for (int e = 0; e < V; ++e) y[e] += h[e] * a.w[(size_t)(c + e) * taps + taps - 1];
+    }
+    if (taps > 1) store_v<float, V>(next + (size_t)(taps - 2) * D, h);
+#pragma unroll
+    for (int e = 0; e < V; ++e) y[e] += h[e];
+    if (!a.mu) {
+      store_v<T, V>(out, y);
+      return;
+    }
+    store_v<float, V>(p_next, y);
+    auto blend = [&](int i, const float (&m)[V]) {
+      float v[V];
+#pragma unroll
+      for (int e = 0; e < V; ++e) v[e] = y[e] + (prev[e] - y[e]) * m[e];
+      store_v<T, V>(out + i * a.mix_stride, v);
+    };
+    if (small) {
+#pragma unroll
+      for (int i = 0; i < MAX_MIX; ++i)
+        if (i < a.n_mix) blend(i, mu[i]);
+    } else {
+      for (int i = 0; i < a.n_mix; ++i) {
+        float m[V];
+        load_v<float, V>(a.mu + (size_t)i * D + c, true, m);
+        blend(i, m);
+      }
+    }
+  }
+};
+// the sum of `parts` rows
+template <int V>
+DEV void load_sum(const float* p, bool in, int parts, size_t stride, float (&v)[V]) {
+  load_v<float, V>(p, in, v);
+  for (int k = 1; k < parts; k += 4) {
+    float q[4][V];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) load_v<float, V>(p + (k + u) * stride, in && k + u < parts, q[u]);
+#pragma unroll
+    for (int u = 0; u < 4; ++u)
+#pragma unroll
+      for (int e = 0; e < V; ++e) v[e] += q[u][e];
+  }
 }
-template <typename T, int NT, int VPT, int V>
+template <typename T, int NT, int VPT, int V, bool CONV>
 __global__ __launch_bounds__(NT) void join_kernel(const JoinArgs a) {
   __shared__ float red[NT / 64], s_w[64];
   __shared__ int s_pos[64];
@@ -82,6 +134,17 @@ __global__ __launch_bounds__(NT) void join_kernel(const JoinArgs a) {
   const int hrow = blockIdx.x;
   float x[VPT][V], add[VPT][V];
   auto at = [&](int i) { return V * (tid + i * NT); };
+  // with a convolution behind the norm: everything it reads, requested first (one group per thread) or together with its use (more)
+  ConvOne<V> cv;
+  SeqDesc sq{};
+  float nw[V];
+  if constexpr (CONV) {
+    sq = a.p.seqs[a.p.row_seq[row]];
+    if constexpr (VPT == 1) {
+      cv.load(a, sq, at(0));
+      load_v<float, V>(a.norm_w + at(0), at(0) < D, nw);
+    }
+  }
   if (a.y_t && tid < a.n_slots) {
     s_w[tid] = a.weight[(size_t)row * a.n_slots + tid];
     s_pos[tid] = a.slot_pos[(size_t)row * a.n_slots + tid];
@@ -96,13 +159,13 @@ __global__ __launch_bounds__(NT) void join_kernel(const JoinArgs a) {
   if (a.mix_a) {
     const float* ma = a.mix_a + (size_t)row * a.mix_ld;
 #pragma unroll
-    for (int i = 0; i < VPT; ++i) load_v<float, V>(ma + at(i), at(i) < D, add[i]);
+    for (int i = 0; i < VPT; ++i) load_sum<V>(ma + at(i), at(i) < D, a.parts_a, a.mix_stride, add[i]);
     if (a.mix_b) {
       const float* mb = a.mix_b + (size_t)row * a.mix_ld;
       float vb[VPT][V], sa = 0.f, sb = 0.f;
 #pragma unroll
       for (int i = 0; i < VPT; ++i) {
-        load_v<float, V>(mb + at(i), at(i) < D, vb[i]);
+        load_sum<V>(mb + at(i), at(i) < D, a.parts_b, a.mix_stride, vb[i]);
 #pragma unroll
         for (int e = 0; e < V; ++e) {
           sa += add[i][e] * add[i][e];
@@ -170,18 +233,24 @@ __global__ __launch_bounds__(NT) void join_kernel(const JoinArgs a) {
   for (int i = 0; i < VPT; ++i) {
     if (at(i) >= D) continue;
     float w[V];
-    load_v<float, V>(a.norm_w + at(i), true, w);
+    if constexpr (CONV && VPT == 1) {
+#pragma unroll
+      for (int e = 0; e < V; ++e) w[e] = nw[e];
+    } else {
+      if constexpr (CONV) cv.load(a, sq, at(i));
+      load_v<float, V>(a.norm_w + at(i), true, w);
+    }
 #pragma unroll
     for (int e = 0; e < V; ++e) w[e] = x[i][e] * r * (w[e] + a.norm_offset);
-    if (a.conv.w) conv_one<T, V>(a, row, at(i), w);
+    if constexpr (CONV) cv.template run<T>(a, row, sq.pos0, at(i), w);
     else if (a.h_f) store_v<float, V>(a.h_f + (size_t)row * D + at(i), w);
     else store_v<T, V>(h + at(i), w);
   }
 }
-template <typename T>
+template <typename T, bool CONV>
 static int join_t(hipStream_t st, const JoinArgs& a, int n) {
   const int D = a.width;
-#define JOIN(NT, VPT, V) hipLaunchKernelGGL((join_kernel<T, NT, VPT, V>), dim3(n), dim3(NT), 0, st, a)
+#define JOIN(NT, VPT, V) hipLaunchKernelGGL((join_kernel<T, NT, VPT, V, CONV>), dim3(n), dim3(NT), 0, st, a)
   if (D > 16384) DSK_FAIL(DSK_ERR_UNSUPPORTED, "join: width %d (max 16384)", D);
   if (D & 3) {
     if (D <= 1024) JOIN(256, 4, 1);
@@ -198,10 +267,27 @@ static int join_t(hipStream_t st, const JoinArgs& a, int n) {
 int launch_join(hipStream_t st, const JoinArgs& a, bool f32) {
   const int n = a.only_want ? a.p.n_want : a.p.rows;
   if (n < 1) DSK_FAIL(DSK_ERR_INVALID, "join: no rows");
-  return f32 ? join_t<float>(st, a, n) : join_t<bf16>(st, a, n);
+  if (a.conv.w) return f32 ? join_t<float, true>(st, a, n) : join_t<bf16, true>(st, a, n);
+  return f32 ? join_t<float, false>(st, a, n) : join_t<bf16, false>(st, a, n);
 }
 
 // ---- convolution in front of a sublayer, portions --------------------------------------------------------
+// y, or its blends with the previous token's y, of V channels from c on
+template <typename T, int V>
+DEV void store_blends(const ConvArgs& a, int D, int row, int c, const float (&y)[V], const float (&prev)[V]) {
+  T* out = reinterpret_cast<T*>(a.out_t) + (size_t)row * a.ld + c;
+  if (!a.mu) {
+    store_v<T, V>(out, y);
+    return;
+  }
+  for (int s = 0; s < a.n_mix; ++s) {
+    float m[V];
+    load_v<float, V>(a.mu + (size_t)s * D + c, true, m);
+#pragma unroll
+    for (int e = 0; e < V; ++e) m[e] = y[e] + (prev[e] - y[e]) * m[e];
+    store_v<T, V>(out + s * a.mix_stride, m);
+  }
+}
 // A thread takes V channels of the (up to 16) rows of a chunk; TAPS = 0: any number of taps, read from memory again and again.
 template <typename T, int V, int TAPS>
 __global__ __launch_bounds__(256) void conv_kernel(const PassDesc p, int D, const float* __restrict__ h_f, const ConvArgs a) {

@@ -35,32 +35,63 @@ DEV float turned(X x, const float* turn, int rot_dims, int j) {
 }
 
 // ---- norms and rotation: one workgroup per row --------------------------------------------------------------
+enum { PREP_NT = 512 };
 template <typename T>
-__global__ __launch_bounds__(256) void latent_prep_kernel(const LatentArgs a) {
-  __shared__ float red[4];
+__global__ __launch_bounds__(PREP_NT) void latent_prep_kernel(const LatentArgs a) {
+  constexpr int NT = PREP_NT, U = 4;  // U elements of either latent per thread wait in registers; larger ones are read again
+  __shared__ float red[2 * NT / 64];
   const int row = blockIdx.x, tid = threadIdx.x, half = a.rot_dims >> 1, ld = a.rank_p + a.rot_p;
   const SeqDesc s = a.p.seqs[a.p.row_seq[row]];
   const int pos = s.pos0 + row - s.row0;
   const float *q = a.proj_f + (size_t)row * a.ld + a.col_q, *kv = a.proj_f + (size_t)row * a.ld + a.col_kv;
-  float sq = 0.f, sk = 0.f;
-  for (int i = tid; i < a.q_rank; i += 256) sq += q[i] * q[i];
-  for (int i = tid; i < a.kv_rank; i += 256) sk += kv[i] * kv[i];
-  sq = block_sum<256>(sq, red);
-  sk = block_sum<256>(sk, red);
-  const float rq = 1.f / sqrtf(sq / a.q_rank + a.eps), rk = 1.f / sqrtf(sk / a.kv_rank + a.eps);
-  T* cq = reinterpret_cast<T*>(a.cq_t) + (size_t)row * a.cq_ld;
-  for (int i = tid; i < a.cq_ld; i += 256) cq[i] = (T)(i < a.q_rank ? q[i] * rq * a.q_norm[i] : 0.f);
-  T* lat = s.len == 1 ? reinterpret_cast<T*>(s.state + a.off_c) + (size_t)(pos % a.window) * ld : reinterpret_cast<T*>(a.lat_t) + (size_t)(s.key0 + s.hist + row - s.row0) * ld;
-  for (int i = tid; i < a.rank_p; i += 256) lat[i] = (T)(i < a.kv_rank ? kv[i] * rk * a.kv_norm[i] : 0.f);
+  float xq[U], xk[U], wq[U], wk[U], sq = 0.f, sk = 0.f;
+#pragma unroll
+  for (int u = 0; u < U; ++u) {
+    const int i = tid + u * NT;
+    xq[u] = i < a.q_rank ? q[i] : 0.f;
+    wq[u] = i < a.q_rank ? a.q_norm[i] : 0.f;
+    xk[u] = i < a.kv_rank ? kv[i] : 0.f;
+    wk[u] = i < a.kv_rank ? a.kv_norm[i] : 0.f;
+  }
   float* turn = a.turn + (size_t)row * a.rot_dims;
-  for (int i = tid; i < half; i += 256) {
+  for (int i = tid; i < half; i += NT) {
     float sn, cs;
     sincosf((float)pos * a.freq[i], &sn, &cs);
     turn[i] = cs;
     turn[half + i] = sn;
   }
-  __syncthreads();  // (this workgroup's own stores: visible to it behind the barrier)
-  for (int j = tid; j < a.rot_p; j += 256) lat[a.rank_p + j] = (T)(j < a.rot_dim ? turned([&](int i) { return kv[a.kv_rank + i]; }, turn, a.rot_dims, j) : 0.f);
+#pragma unroll
+  for (int u = 0; u < U; ++u) {
+    sq += xq[u] * xq[u];
+    sk += xk[u] * xk[u];
+  }
+  for (int i = tid + U * NT; i < a.q_rank; i += NT) sq += q[i] * q[i];
+  for (int i = tid + U * NT; i < a.kv_rank; i += NT) sk += kv[i] * kv[i];
+  sq = wave_sum(sq);
+  sk = wave_sum(sk);
+  if ((tid & 63) == 0) {
+    red[tid >> 6] = sq;
+    red[NT / 64 + (tid >> 6)] = sk;
+  }
+  __syncthreads();  // (the cosines and sines too: this workgroup's own stores are visible to it behind the barrier)
+  sq = sk = 0.f;
+#pragma unroll
+  for (int i = 0; i < NT / 64; ++i) {
+    sq += red[i];
+    sk += red[NT / 64 + i];
+  }
+  const float rq = 1.f / sqrtf(sq / a.q_rank + a.eps), rk = 1.f / sqrtf(sk / a.kv_rank + a.eps);
+  T* cq = reinterpret_cast<T*>(a.cq_t) + (size_t)row * a.cq_ld;
+  T* lat = s.len == 1 ? reinterpret_cast<T*>(s.state + a.off_c) + (size_t)(pos % a.window) * ld : reinterpret_cast<T*>(a.lat_t) + (size_t)(s.key0 + s.hist + row - s.row0) * ld;
+#pragma unroll
+  for (int u = 0; u < U; ++u) {
+    const int i = tid + u * NT;
+    if (i < a.cq_ld) cq[i] = (T)(xq[u] * rq * wq[u]);
+    if (i < a.rank_p) lat[i] = (T)(xk[u] * rk * wk[u]);
+  }
+  for (int i = tid + U * NT; i < a.cq_ld; i += NT) cq[i] = (T)(i < a.q_rank ? q[i] * rq * a.q_norm[i] : 0.f);
+  for (int i = tid + U * NT; i < a.rank_p; i += NT) lat[i] = (T)(i < a.kv_rank ? kv[i] * rk * a.kv_norm[i] : 0.f);
+  for (int j = tid; j < a.rot_p; j += NT) lat[a.rank_p + j] = (T)(j < a.rot_dim ? turned([&](int i) { return kv[a.kv_rank + i]; }, turn, a.rot_dims, j) : 0.f);
 }
 
 // ---- rows between ring and key workspace -----------------------------------------------------------------------
@@ -125,10 +156,10 @@ struct LatentKeys {
 };
 template <typename T, int KT, int VTL>
 __global__ __launch_bounds__(256) void latent_attn_kernel(const LatentArgs a) {
-  const int h = blockIdx.y;
-  const SeqDesc s = a.p.seqs[a.p.qtile[2 * blockIdx.x]];
+  const int h = blockIdx.y, tile = gridDim.x - 1 - blockIdx.x;  // (a sequence's last tiles have the most keys: they start first)
+  const SeqDesc s = a.p.seqs[a.p.qtile[2 * tile]];
   if (s.len == 1) return;
-  attn_tile<T, KT, VTL>(LatentKeys<T>{a, s, h}, s, a.p.qtile[2 * blockIdx.x + 1], (a.dim_p + a.rot_p) >> 5, a.vdim_p >> 4, a.vdim, a.scale,
+  attn_tile<T, KT, VTL>(LatentKeys<T>{a, s, h}, s, a.p.qtile[2 * tile + 1], (a.dim_p + a.rot_p) >> 5, a.vdim_p >> 4, a.vdim, a.scale,
                         reinterpret_cast<T*>(a.out_t) + h * a.vdim, a.out_ld);
 }
 
@@ -156,11 +187,20 @@ __global__ __launch_bounds__(FEW_NT) void latent_few_kernel(const LatentArgs a) 
   T* pw = reinterpret_cast<T*>(red + FEW_NW * 64);        // [16][LP] weights
   const T* ring = reinterpret_cast<const T*>(s.state + a.off_c);
   const int ng = ld >> 3, first = pos - seen + 1 + k0;
-  for (int u = tid; u < N * ng; u += FEW_NT) {
-    const int key = u / ng, gr = u % ng;
-    frag f = frag{};
-    if (key < n) f = *reinterpret_cast<const frag*>(ring + (size_t)((first + key) % a.window) * ld + gr * 8);
-    *reinterpret_cast<frag*>(lat + (size_t)key * LD + gr * 8) = f;
+  constexpr int IN_FLIGHT = sizeof(T) == 2 ? 12 : 6;
+  for (int u0 = tid; u0 < N * ng; u0 += FEW_NT * IN_FLIGHT) {
+    frag f[IN_FLIGHT];
+#pragma unroll
+    for (int j = 0; j < IN_FLIGHT; ++j) {
+      const int u = u0 + j * FEW_NT, key = u / ng, gr = u % ng;
+      f[j] = frag{};
+      if (key < n) f[j] = *reinterpret_cast<const frag*>(ring + (size_t)((first + key) % a.window) * ld + gr * 8);
+    }
+#pragma unroll
+    for (int j = 0; j < IN_FLIGHT; ++j) {
+      const int u = u0 + j * FEW_NT;
+      if (u < N * ng) *reinterpret_cast<frag*>(lat + (size_t)(u / ng) * LD + u % ng * 8) = f[j];
+    }
   }
   const float* turn = a.turn + (size_t)s.row0 * a.rot_dims;
   const int hd = a.dim_p + a.rot_p;
@@ -234,6 +274,15 @@ __global__ __launch_bounds__(256) void latent_values_kernel(const LatentArgs a) 
   float* c = reinterpret_cast<float*>(lds);  // [rank_p] merged latent
   float* w = c + a.rank_p;                   // [splits] weights of the parts
   float* red = w + (a.splits + 3) / 4 * 4;   // [4][64]
+  const int r = v0 + lane, R = a.up_row + h * a.vdim_p + min(r, a.vdim_p - 1), ng = a.rank_p >> 3;
+  const bf16* W = reinterpret_cast<const bf16*>(a.up_w) + (size_t)(R >> 4) * a.up_kt * 512 + (R & 15) * 8;
+  constexpr int AHEAD = 16;                  // this thread's first weights, requested before anything else
+  bf16x8 x[AHEAD];
+#pragma unroll
+  for (int u = 0; u < AHEAD; ++u) {
+    const int gr = min(wave + 4 * u, ng - 1);
+    x[u] = *reinterpret_cast<const bf16x8*>(W + (size_t)(gr >> 2) * 512 + (gr & 3) * 128);
+  }
   const float* ml = a.part_ml + ((size_t)i * a.heads + h) * a.splits * 2;
   float m = -INFINITY, l = 0.f;              // (every wave for itself)
   for (int k = lane; k < n; k += 64) m = fmaxf(m, ml[2 * k]);
@@ -247,21 +296,32 @@ __global__ __launch_bounds__(256) void latent_values_kernel(const LatentArgs a) 
   l = wave_sum(l);
   __syncthreads();
   const float* part = a.part + ((size_t)i * a.heads + h) * a.splits * a.rank_p;
-  for (int e = tid; e < a.rank_p; e += 256) {
-    float o = 0.f;
-#pragma unroll 8
-    for (int k = 0; k < n; ++k) o += w[k] * part[(size_t)k * a.rank_p + e];
-    c[e] = (float)(T)(o / l);
+  for (int e = tid * 4; e < a.rank_p; e += 1024) {
+    f32x4 o = {0.f, 0.f, 0.f, 0.f};
+    for (int k0 = 0; k0 < n; k0 += 8) {
+      f32x4 v[8];
+#pragma unroll
+      for (int u = 0; u < 8; ++u) v[u] = *reinterpret_cast<const f32x4*>(part + (size_t)min(k0 + u, n - 1) * a.rank_p + e);
+#pragma unroll
+      for (int u = 0; u < 8; ++u)
+        if (k0 + u < n) o += w[k0 + u] * v[u];
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) c[e + j] = (float)(T)(o[j] / l);
   }
   __syncthreads();
-  const int r = v0 + lane, R = a.up_row + h * a.vdim_p + min(r, a.vdim_p - 1);
-  const bf16* W = reinterpret_cast<const bf16*>(a.up_w) + (size_t)(R >> 4) * a.up_kt * 512 + (R & 15) * 8;
   float z = 0.f;
-#pragma unroll 8
-  for (int gr = wave; gr < a.rank_p >> 3; gr += 4) {
-    const bf16x8 x = *reinterpret_cast<const bf16x8*>(W + (size_t)(gr >> 2) * 512 + (gr & 3) * 128);
 #pragma unroll
-    for (int e = 0; e < 8; ++e) z += (float)x[e] * c[gr * 8 + e];
+  for (int u = 0; u < AHEAD; ++u) {
+    const int gr = wave + 4 * u;
+    if (gr < ng)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) z += (float)x[u][e] * c[gr * 8 + e];
+  }
+  for (int gr = wave + 4 * AHEAD; gr < ng; gr += 4) {
+    const bf16x8 y = *reinterpret_cast<const bf16x8*>(W + (size_t)(gr >> 2) * 512 + (gr & 3) * 128);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) z += (float)y[e] * c[gr * 8 + e];
   }
   red[wave * 64 + lane] = z;
   __syncthreads();
@@ -277,8 +337,8 @@ static int check_latent(const LatentArgs& a, bool f32) {
 }
 int launch_latent_prep(hipStream_t st, const LatentArgs& a, bool f32) {
   DSK_TRY(check_latent(a, f32));
-  if (f32) hipLaunchKernelGGL(latent_prep_kernel<float>, dim3(a.p.rows), dim3(256), 0, st, a);
-  else hipLaunchKernelGGL(latent_prep_kernel<bf16>, dim3(a.p.rows), dim3(256), 0, st, a);
+  if (f32) hipLaunchKernelGGL(latent_prep_kernel<float>, dim3(a.p.rows), dim3(PREP_NT), 0, st, a);
+  else hipLaunchKernelGGL(latent_prep_kernel<bf16>, dim3(a.p.rows), dim3(PREP_NT), 0, st, a);
   return DSK_OK;
 }
 int launch_latent_gather(hipStream_t st, const LatentArgs& a, bool f32) {

@@ -10,6 +10,8 @@
 
 #include <math.h>
 
+#include <algorithm>
+
 typedef const __attribute__((address_space(1))) void* gptr;
 typedef __attribute__((address_space(3))) void* lptr;
 
@@ -82,7 +84,8 @@ DEV void store_plain(const LinArgs& a, int row, int feature, f32x4 v) {
     v *= a.p0;
   } else if (a.epi == LIN_XIELU) {
 #pragma unroll
-    for (int i = 0; i < 4; ++i) v[i] = 0.5f * v[i] + (v[i] > 0.f ? a.p0 * v[i] * v[i] : a.p1 * (expm1f(v[i]) - v[i]));
+    for (int i = 0; i < 4; ++i)  // (exp(z) - 1 - z: its absolute error is a rounding of 1, and z / 2 is beside it)
+      v[i] = 0.5f * v[i] + (v[i] > 0.f ? a.p0 * v[i] * v[i] : a.p1 * (__expf(fminf(v[i], 0.f)) - 1.f - v[i]));
   } else if (a.epi == LIN_TANH_F && feature >= a.n_wide) {
 #pragma unroll
     for (int i = 0; i < 4; ++i) v[i] = tanhf(v[i]);
@@ -99,6 +102,8 @@ DEV void store_glu(const LinArgs& a, int row, int feature, const f32x4& g, const
   *reinterpret_cast<four*>(reinterpret_cast<T*>(a.out_t) + (size_t)row * a.ld_t + feature) = to_four<T>(v);
 }
 
+// k tiles per part: even, so that a part is whole steps of the prompt kernel
+__host__ DEV int part_tiles(const LinArgs& a) { return a.parts > 1 ? ((a.kt / 2 + a.parts - 1) / a.parts) * 2 : a.kt; }
 // the operand a product's features from `feature` on read
 template <typename T>
 DEV const T* operand(const LinArgs& a, int feature) {
@@ -110,7 +115,7 @@ DEV const T* operand(const LinArgs& a, int feature) {
 // grid.x: row tiles of 128 (experts: entries of the tile table), grid.y: feature tiles of 128.
 // rows: a gather table (slot -> row) or nullptr; out rows are row0 + local row.
 template <typename T>
-DEV void lin_body(const LinArgs& a, const int* gather, int row0, int n_rows, int f0, char* lds) {
+DEV void lin_body(const LinArgs& a, const int* gather, int row0, int n_rows, int f0, int k0, int k1, char* lds) {
   typedef typename Frag<T>::type frag;
   constexpr int AB = 64 * (int)sizeof(frag);  // bytes of an A fragment
   constexpr int STAGE = 16 * 1024 + 16 * AB;  // 8 row tiles x 2 k tiles of each operand
@@ -158,12 +163,12 @@ DEV void lin_body(const LinArgs& a, const int* gather, int row0, int n_rows, int
   for (int i = 0; i < 4; ++i)
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-  stage(0, lds);
-  for (int kt = 0; kt < a.kt; kt += 2) {
+  stage(k0, lds);
+  for (int kt = k0; kt < k1; kt += 2) {
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this wave's loads into LDS; the barrier makes it everybody's
     __syncthreads();
     char* cur = lds + ((kt >> 1) & 1) * STAGE;
-    if (kt + 2 < a.kt) stage(kt + 2, lds + (((kt >> 1) & 1) ^ 1) * STAGE);
+    if (kt + 2 < k1) stage(kt + 2, lds + (((kt >> 1) & 1) ^ 1) * STAGE);
 #pragma unroll
     for (int kk = 0; kk < 2; ++kk) {
       bf16x8 w[4];
@@ -195,10 +200,11 @@ DEV void lin_body(const LinArgs& a, const int* gather, int row0, int n_rows, int
   }
 }
 template <typename T>
-__global__ __launch_bounds__(256) void lin_kernel(const LinArgs a) {
+__global__ __launch_bounds__(256) void lin_kernel(LinArgs a) {
   extern __shared__ __attribute__((aligned(16))) char lds[];
-  const int row0 = blockIdx.x * 128;
-  lin_body<T>(a, nullptr, row0, min(128, a.rows - row0), blockIdx.y * 128, lds);
+  const int row0 = blockIdx.x * 128, per = part_tiles(a), k0 = blockIdx.z * per;
+  a.out_f += blockIdx.z * a.part_stride;
+  lin_body<T>(a, nullptr, row0, min(128, a.rows - row0), blockIdx.y * 128, k0, min(a.kt, k0 + per), lds);
 }
 
 static LinArgs expert_lin(const MoeArgs& m, bool down) {  // the parts of an expert product that do not depend on the expert
@@ -227,35 +233,35 @@ __global__ __launch_bounds__(256) void expert_kernel(LinArgs a, const MoeArgs m,
   const int expert = m.tiles[4 * blockIdx.x], s0 = m.tiles[4 * blockIdx.x + 1], n = m.tiles[4 * blockIdx.x + 2];
   set_expert(a, m, down ? m.down : m.up, expert);
   if ((int)blockIdx.y * 8 >= a.rt) return;
-  lin_body<T>(a, down ? nullptr : m.slot_row, s0, n, blockIdx.y * 128, lds);
+  lin_body<T>(a, down ? nullptr : m.slot_row, s0, n, blockIdx.y * 128, 0, a.kt, lds);
 }
 
 // ---- up to 16 rows -------------------------------------------------------------------------------
 // One workgroup = 16 features (32 with a gate / up pair): wave w takes k tiles w, w + 4, ...; partial sums meet in LDS.
 // row_of: A row of this lane's column; keep: out row or -1.
 template <typename T, int NR>
-DEV void few_body(const LinArgs& a, int rt0, int a_row, int out_row, float* lds) {
+DEV void few_body(const LinArgs& a, int rt0, int k_first, int k_end, int a_row, int out_row, float* lds) {
   typedef typename Frag<T>::type frag;
-  constexpr int U = 4;
+  constexpr int U = NR == 1 && sizeof(T) == 2 ? 8 : 4;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const bf16x8* w0 = reinterpret_cast<const bf16x8*>(a.w) + (size_t)rt0 * a.kt * 64 + lane;
   const T* x0 = operand<T>(a, rt0 * 16) + (size_t)a_row * a.lda + (lane >> 4) * 8;
   f32x4 acc[NR];
 #pragma unroll
   for (int i = 0; i < NR; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-  for (int k0 = wave; k0 < a.kt; k0 += 4 * U) {
+  for (int k0 = k_first + wave; k0 < k_end; k0 += 4 * U) {
     bf16x8 w[U][NR];
     frag x[U];
 #pragma unroll
     for (int u = 0; u < U; ++u) {
-      const int k = min(k0 + 4 * u, a.kt - 1);
+      const int k = min(k0 + 4 * u, k_end - 1);
 #pragma unroll
       for (int i = 0; i < NR; ++i) w[u][i] = w0[((size_t)i * a.kt + k) * 64];
       x[u] = *reinterpret_cast<const frag*>(x0 + (size_t)k * 32);
     }
 #pragma unroll
     for (int u = 0; u < U; ++u)
-      if (k0 + 4 * u < a.kt)
+      if (k0 + 4 * u < k_end)
 #pragma unroll
         for (int i = 0; i < NR; ++i) acc[i] = mma(w[u][i], x[u], acc[i]);
   }
@@ -300,23 +306,25 @@ __global__ __launch_bounds__(256) void few_kernel(const FewArgs f) {
     const int slot = f.m.active_slot[i * 16 + row];
     const int pos = row * (f.m.top + f.m.shared) + max(slot, 0);
     const int out = c < f.m.rows && slot >= 0 ? pos : -1;
-    if (f.down) few_body<T, 1>(a, tile, pos, out, lds);
-    else few_body<T, 2>(a, tile * 2, row, out, lds);
+    if (f.down) few_body<T, 1>(a, tile, 0, a.kt, pos, out, lds);
+    else few_body<T, 2>(a, tile * 2, 0, a.kt, row, out, lds);
     return;
   }
   b -= f.expert_wgs;
   int i = 0;
   while (i + 1 < f.n && b >= f.wg_end[i]) ++i;
-  const LinArgs& a = f.t[i];
+  LinArgs a = f.t[i];
   if (i > 0) b -= f.wg_end[i - 1];
-  const int row = min(c, a.rows - 1);
-  few_body<T, 1>(a, b, a.row_seq ? a.seqs[a.row_seq[row]].row0 : row, c < a.rows ? c : -1, lds);
+  const int row = min(c, a.rows - 1), part = b / a.rt, per = part_tiles(a);
+  a.out_f += part * a.part_stride;
+  few_body<T, 1>(a, b % a.rt, part * per, min(a.kt, part * per + per), a.row_seq ? a.seqs[a.row_seq[row]].row0 : row, c < a.rows ? c : -1, lds);
 }
 
 // ---- launches ------------------------------------------------------------------------------------
 static int lin_lds(bool f32) { return 2 * (16 * 1024 + 16 * 64 * (f32 ? 32 : 16)); }
 static int check_lin(const LinArgs& a, const char* what) {
   if (!a.w || !a.a_t || a.rows < 1 || a.kt < 2 || (a.kt & 1) || a.rt < 1 || a.lda < a.kt * 32) DSK_FAIL(DSK_ERR_INVALID, "%s: rows %d kt %d rt %d lda %d", what, a.rows, a.kt, a.rt, a.lda);
+  if (a.parts > 1 && (a.n_wide || a.epi != LIN_STORE || part_tiles(a) * (a.parts - 1) >= a.kt)) DSK_FAIL(DSK_ERR_INVALID, "%s: %d parts of %d", what, a.parts, a.kt);
   if (a.a_seg < 0 || (a.a_seg & 15) || (a.a_seg && a.a_ops < 1)) DSK_FAIL(DSK_ERR_INVALID, "%s: %d features per operand", what, a.a_seg);
   return DSK_OK;
 }
@@ -328,7 +336,7 @@ static int allow_lds(K k, int bytes) {
 int launch_lin(hipStream_t st, const LinArgs& a, bool f32) {
   DSK_TRY(check_lin(a, "lin"));
   if ((a.a_seg & 127) || a.row_seq) DSK_FAIL(DSK_ERR_INVALID, "lin: %d features per operand", a.a_seg);
-  const dim3 grid(cdiv(a.rows, 128), cdiv(a.rt, 8));
+  const dim3 grid(cdiv(a.rows, 128), cdiv(a.rt, 8), std::max(a.parts, 1));
   const int lds = lin_lds(f32);
   if (f32) {
     DSK_TRY(allow_lds(lin_kernel<float>, lds));
@@ -361,7 +369,7 @@ static int launch_few(hipStream_t st, FewArgs& f, const LinArgs* a, int n, bool 
     DSK_TRY(check_lin(a[i], "lin_few"));
     if (a[i].rows > 16) DSK_FAIL(DSK_ERR_INVALID, "lin_few: %d rows", a[i].rows);
     f.t[i] = a[i];
-    f.wg_end[i] = wgs += a[i].rt;
+    f.wg_end[i] = wgs += a[i].rt * std::max(a[i].parts, 1);
   }
   const dim3 grid(f.expert_wgs + wgs);
   if (f32) hipLaunchKernelGGL(few_kernel<float>, grid, dim3(256), 0, st, f);

@@ -57,6 +57,8 @@ struct LinArgs {
                           // LIN_SCALE: the factor; LIN_XIELU: z > 0: p0 z^2 + z / 2, else p1 (exp(z) - 1 - z) + z / 2; LIN_TANH_F: tanh of the 32-bit part
   int a_seg, a_ops;       // a_seg > 0: features [i a_seg, (i + 1) a_seg) read operand i (the last one: the rest) of a_ops ...
   size_t a_stride;        // ... a_stride elements behind each other (launch_lin: a_seg is a multiple of 128, else of 16)
+  int parts;              // > 1: k in `parts` ranges, each with a 32-bit output of its own (part_stride elements behind each other; n_wide = 0,
+  size_t part_stride;     // LIN_STORE); the reader adds them up
   const int* row_seq;     // launch_lin_few: output row i reads the first row of sequence row_seq[i] of seqs (nullptr: row i)
   const SeqDesc* seqs;
 };
@@ -124,6 +126,8 @@ struct JoinArgs {           // x += (what the previous layer left); h = norm(x)
   float* x;                 // [rows][width]
   const uint16_t* embed;    // first layer: x = embed[token] (nothing to add)
   const float* mix_a;       // mixer output [rows][mix_ld] (nullptr: none)
+  int parts_a, parts_b;     // mix_a (mix_b) is the sum of this many, mix_stride elements behind each other
+  size_t mix_stride;
   const float* mix_b;       // second of a pair: half the sum of both, each RMS-normed with its weight
   int mix_ld;
   const float *pair_wa, *pair_wb;

@@ -15,7 +15,7 @@
 
 namespace {
 
-enum { FEW = 16, LOGIT_ROWS = 128 };
+enum { FEW = 16, LOGIT_ROWS = 128, MIX_PARTS = 4, MIX_PARTS_FEW = 8 };
 
 size_t up(size_t v, size_t a) { return (v + a - 1) / a * a; }
 
@@ -109,6 +109,8 @@ struct LayeredModel : ModelHead {
   float* x = nullptr;
   char *h = nullptr, *hw = nullptr, *wide = nullptr, *out_a = nullptr, *out_b = nullptr, *qb = nullptr, *kb = nullptr, *vb = nullptr, *hidden = nullptr, *y = nullptr;
   float *narrow = nullptr, *mix_a = nullptr, *mix_b = nullptr, *low = nullptr, *dq = nullptr, *dk = nullptr, *dv = nullptr, *dg = nullptr, *db = nullptr, *o = nullptr;
+  int mix_parts[2] = {1, 1};        // of the products that wrote mix_a and mix_b last
+  size_t mix_stride = 0;
   // sandwich layers, latent attention
   float *h_f = nullptr, *turn = nullptr, *lat_part = nullptr, *lat_ml = nullptr;
   char *cq = nullptr, *lq = nullptr, *lat = nullptr, *kv = nullptr, *qabs = nullptr;
@@ -601,8 +603,9 @@ int alloc_work(LayeredModel* m) {
   DSK_TRY(dev_alloc_n(m, &m->narrow, n * m->ldf));
   DSK_TRY(dev_alloc(m, (void**)&m->out_a, n * m->out_ld * e));
   DSK_TRY(dev_alloc(m, (void**)&m->out_b, n * m->out_ld * e));
-  DSK_TRY(dev_alloc_n(m, &m->mix_a, n * m->mix_ld));
-  DSK_TRY(dev_alloc_n(m, &m->mix_b, n * m->mix_ld));
+  const size_t mix_rows = std::max<size_t>(n * MIX_PARTS, FEW * MIX_PARTS_FEW);
+  DSK_TRY(dev_alloc_n(m, &m->mix_a, mix_rows * m->mix_ld));
+  DSK_TRY(dev_alloc_n(m, &m->mix_b, mix_rows * m->mix_ld));
   DSK_TRY(dev_alloc(m, (void**)&m->qb, n * aq * e));
   DSK_TRY(dev_alloc(m, (void**)&m->kb, n * ak * e));
   DSK_TRY(dev_alloc(m, (void**)&m->vb, n * av * e));
@@ -669,6 +672,16 @@ LinArgs lin_f(const PackedMat& w, const void* a, int lda, int rows, float* out, 
   l.ld_f = ld;
   return l;
 }
+// A product whose output the next residual sum reads (mix_a; second: mix_b), split over k where its tiles alone leave compute units idle
+LinArgs mix_lin(LayeredModel* m, const PackedMat& w, const void* a, int lda, int rows, bool few, bool second = false) {
+  const int tiles = few ? w.rt : ((rows + 127) / 128) * ((w.rt + 7) / 8);
+  const int n = std::max(std::min({few ? 1024 / tiles : 512 / tiles, w.kt / 16, (int)(few ? MIX_PARTS_FEW : MIX_PARTS)}), 1);
+  const int per = (w.kt / 2 + n - 1) / n * 2;  // (no part may be empty)
+  LinArgs l = lin_f(w, a, lda, rows, second ? m->mix_b : m->mix_a, m->mix_ld);
+  l.parts = m->mix_parts[second] = (w.kt + per - 1) / per;
+  l.part_stride = m->mix_stride = (size_t)rows * m->mix_ld;
+  return l;
+}
 int run_lin(LayeredModel* m, const LinArgs* a, int n, bool few) {
   if (few) return launch_lin_few(m->ctx->stream, a, n, m->f32);
   for (int i = 0; i < n; ++i) DSK_TRY(launch_lin(m->ctx->stream, a[i], m->f32));
@@ -693,6 +706,9 @@ JoinArgs join_args(LayeredModel* m, const PassDesc& p, int l) {
   const LayerSpec& s = m->s.layers[l - 1];
   const LayerW& w = m->L[l - 1];
   j.mix_a = m->mix_a;
+  j.parts_a = m->mix_parts[0];
+  j.parts_b = m->mix_parts[1];
+  j.mix_stride = m->mix_stride;
   j.post_w = s.has_dense ? w.ff_post : w.post;
   if (w.pair_a) {
     j.mix_b = m->mix_b;
@@ -1036,22 +1052,22 @@ int run_layer(LayeredModel* m, const PassDesc& p, int l, bool few) {
   MixFewArgs f{};
   if (s.has_attn) {
     f.attn = attn_args(m, p, s, w);
-    outs[n_out++] = lin_f(w.a_o, m->out_a, w.a_o.kt * 32, p.rows, m->mix_a, m->mix_ld);
+    outs[n_out++] = mix_lin(m, w.a_o, m->out_a, w.a_o.kt * 32, p.rows, few);
   }
   if (s.has_mlstm) {
     f.mlstm = mlstm_args(m, p, s, w, n_out ? m->out_b : m->out_a);
-    outs[n_out] = lin_f(w.m_o, n_out ? m->out_b : m->out_a, w.m_o.kt * 32, p.rows, n_out ? m->mix_b : m->mix_a, m->mix_ld);
+    outs[n_out] = mix_lin(m, w.m_o, n_out ? m->out_b : m->out_a, w.m_o.kt * 32, p.rows, few, n_out > 0);
     ++n_out;
   }
   if (s.has_delta) {
     f.delta = delta_args(m, p, s, w);
-    outs[n_out++] = lin_f(w.d_o, m->out_a, w.d_o.kt * 32, p.rows, m->mix_a, m->mix_ld);
+    outs[n_out++] = mix_lin(m, w.d_o, m->out_a, w.d_o.kt * 32, p.rows, few);
   }
   if (s.has_wkv) {
     f.wkv = wkv_args(m, p, s, w);
-    outs[n_out++] = lin_f(w.w_o, m->out_a, w.w_o.kt * 32, p.rows, m->mix_a, m->mix_ld);
+    outs[n_out++] = mix_lin(m, w.w_o, m->out_a, w.w_o.kt * 32, p.rows, few);
   }
-  if (s.has_latent) outs[n_out++] = lin_f(w.l_o, m->out_a, w.l_o.kt * 32, p.rows, m->mix_a, m->mix_ld);
+  if (s.has_latent) outs[n_out++] = mix_lin(m, w.l_o, m->out_a, w.l_o.kt * 32, p.rows, few);
   const MoeArgs e = s.has_moe ? moe_args(m, p, s, w) : MoeArgs{};
   f.rows = p.rows;
   f.has_attn = s.has_attn;
@@ -1088,6 +1104,8 @@ int run_layer(LayeredModel* m, const PassDesc& p, int l, bool few) {
     j.embed = nullptr;
     j.y_t = nullptr;
     j.mix_a = m->mix_a;
+    j.parts_a = m->mix_parts[0];
+    j.mix_stride = m->mix_stride;
     j.mix_b = nullptr;
     j.post_w = w.post;
     DSK_TRY(enter(m, j, w.ff_norm, s, w.ff_conv, few));
@@ -1099,7 +1117,7 @@ int run_layer(LayeredModel* m, const PassDesc& p, int l, bool few) {
     u.out_t = m->hidden;
     u.ld_t = m->hid_ld;
     DSK_TRY(run_lin(m, &u, 1, few));
-    const LinArgs d = lin_f(w.ff_down, m->hidden, m->hid_ld, p.rows, m->mix_a, m->mix_ld);
+    const LinArgs d = mix_lin(m, w.ff_down, m->hidden, m->hid_ld, p.rows, few);
     return run_lin(m, &d, 1, few);
   }
   if (!s.has_moe) return run_lin(m, outs, n_out, few);

@@ -43,7 +43,7 @@ DEV void attn_tile(const Keys& src, const SeqDesc& sq, int q0, int kts, int vts,
   typedef typename Frag<T>::type frag;
   typedef typename Frag<T>::four four;
   extern __shared__ __attribute__((aligned(16))) char lds[];
-  constexpr int NS = ATTN_KEYS / 16, KI = KT * NS / 4, VI = (VTL * NS + 15) / 16;  // a thread's share of a tile: KI key groups, VI times 4 keys x 4 channels
+  constexpr int NS = ATTN_KEYS / 16, KI = KT * NS / 4, VI = VTL * NS / 16;  // a wave's share of a tile: KI fragments of keys, VI blocks of values
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int nq = min(64, sq.len - q0);
   T* kf = reinterpret_cast<T*>(lds);                     // fragments of the key tile
@@ -59,21 +59,23 @@ DEV void attn_tile(const Keys& src, const SeqDesc& sq, int q0, int kts, int vts,
   for (int i = 0; i < VTL; ++i) o[i] = f32x4{0.f, 0.f, 0.f, 0.f};
   float m = -INFINITY, l = 0.f;
   const int first = src.first(sq.pos0 + q0), last = sq.pos0 + q0 + nq - 1;
-  const int ng = kts * 4, nv = vts * 4;
+  // A wave loads whole fragments of keys (16 keys x 32 elements: 64 bytes a row, lane-linear in LDS), and blocks of 32 keys x 32 value
+  // channels (8 lanes a row; the transposed writes of 8 rows meet every LDS bank once).
+  const int kr = lane & 15, kg = lane >> 4, vc = (lane & 7) * 4, vk = (lane >> 3) * 4;
   frag rk[KI];
   four rv[VI][4];
   auto fetch = [&](int j0) {  // keys past the tile's last position repeat it (masked below)
 #pragma unroll
     for (int u = 0; u < KI; ++u) {
-      const int i = tid + 256 * u;
-      if (i < ATTN_KEYS * ng) rk[u] = src.k(min(j0 + i / ng, last), i % ng);
+      const int id = wave + 4 * u, kt = id / NS;
+      if (kt < kts) rk[u] = src.k(min(j0 + id % NS * 16 + kr, last), kt * 4 + kg);
     }
 #pragma unroll
     for (int u = 0; u < VI; ++u) {
-      const int i = tid + 256 * u;
-      if (i < ATTN_KEYS / 4 * nv)
+      const int id = wave + 4 * u, c = id / (NS / 2) * 32 + vc;
+      if (c < vts * 16)
 #pragma unroll
-        for (int k = 0; k < 4; ++k) rv[u][k] = src.v(min(j0 + i / nv * 4 + k, last), i % nv * 4);
+        for (int k = 0; k < 4; ++k) rv[u][k] = src.v(min(j0 + id % (NS / 2) * 32 + vk + k, last), c);
     }
   };
   fetch(first);
@@ -81,15 +83,16 @@ DEV void attn_tile(const Keys& src, const SeqDesc& sq, int q0, int kts, int vts,
     __syncthreads();
 #pragma unroll
     for (int u = 0; u < KI; ++u) {
-      const int i = tid + 256 * u, key = i / ng, gr = i % ng;
-      if (i < ATTN_KEYS * ng) *reinterpret_cast<frag*>(kf + (((size_t)(key >> 4) * kts + (gr >> 2)) * 64 + (gr & 3) * 16 + (key & 15)) * 8) = rk[u];
+      const int id = wave + 4 * u, kt = id / NS;
+      if (kt < kts) *reinterpret_cast<frag*>(kf + (((size_t)(id % NS) * kts + kt) * 64 + lane) * 8) = rk[u];
     }
 #pragma unroll
     for (int u = 0; u < VI; ++u) {
-      const int i = tid + 256 * u, kq = i / nv, c = i % nv * 4;
-      if (i < ATTN_KEYS / 4 * nv)
+      const int id = wave + 4 * u, c = id / (NS / 2) * 32 + vc;
+      if (c < vts * 16)
 #pragma unroll
-        for (int e = 0; e < 4; ++e) *reinterpret_cast<four*>(vt + (size_t)(c + e) * VT<T>::LD + kq * 4) = four{rv[u][0][e], rv[u][1][e], rv[u][2][e], rv[u][3][e]};
+        for (int e = 0; e < 4; ++e)
+          *reinterpret_cast<four*>(vt + (size_t)(c + e) * VT<T>::LD + id % (NS / 2) * 32 + vk) = four{rv[u][0][e], rv[u][1][e], rv[u][2][e], rv[u][3][e]};
     }
     __syncthreads();
     if (j0 + ATTN_KEYS <= last) fetch(j0 + ATTN_KEYS);

@@ -28,51 +28,50 @@ DEV void store_v(S* p, const float (&v)[V]) {
     p[0] = (S)v[0];
   }
 }
-// A sequence's only token of the pass: V channels of h through the convolution.  What that needs from memory is requested at once (up to
-// MAX_TAPS taps and MAX_MIX blends; more go one after the other), early enough to be there when h is.
-template <int V>
+// A sequence's only token of the pass: V channels of h through the convolution.  TAPS = 4: what that needs from memory is requested at
+// once, early enough to be there when h is (the blends' weights: up to MAX_MIX); TAPS = 1: any number of taps, one after the other.
+template <int V, int TAPS>
 struct ConvOne {
-  enum { MAX_TAPS = 4, MAX_MIX = 5 };
-  float old[MAX_TAPS - 1][V], w[V][MAX_TAPS], mu[MAX_MIX][V], prev[V];
+  enum { MAX_MIX = 5, KEPT = TAPS > 1 ? TAPS - 1 : 1, MIX = TAPS > 1 ? (int)MAX_MIX : 1 };
+  float old[KEPT][V], w[V * TAPS], mu[MIX][V], prev[V];
   const float* hist;
   float *next, *p_next;
-  bool small;
   DEV void load(const JoinArgs& j, const SeqDesc& s, int c) {
     const ConvArgs& a = j.conv;
-    const int D = j.width, taps = a.taps;
-    const bool in = c < D;
-    small = taps <= MAX_TAPS && a.n_mix <= MAX_MIX;
+    const int D = j.width, taps = TAPS > 1 ? TAPS : a.taps;
     hist = reinterpret_cast<const float*>(s.state + a.off_in) + (size_t)s.flip * (taps - 1) * D + c;
     next = reinterpret_cast<float*>(s.state + a.off_in) + (size_t)(s.flip ^ 1) * (taps - 1) * D + c;
-    float* P = reinterpret_cast<float*>(s.state + a.off_prev) + c;
-    p_next = P + (size_t)(s.flip ^ 1) * D;
-    load_v<float, V>(P + (size_t)s.flip * D, in && a.mu && s.pos0 > 0, prev);
-    if (!small || !in) return;
+    p_next = reinterpret_cast<float*>(s.state + a.off_prev) + c + (size_t)(s.flip ^ 1) * D;
+    if (c >= D) return;
+    if constexpr (TAPS > 1) {
 #pragma unroll
-    for (int t = 0; t < MAX_TAPS - 1; ++t) load_v<float, V>(hist + (size_t)t * D, t < taps - 1 && s.pos0 - (taps - 1) + t >= 0, old[t]);
+      for (int t = 0; t < KEPT; ++t) load_v<float, V>(hist + (size_t)t * D, s.pos0 - (taps - 1) + t >= 0, old[t]);
 #pragma unroll
-    for (int e = 0; e < V; ++e)
+      for (int e = 0; e < TAPS; ++e) load_v<float, V>(a.w + (size_t)c * taps + e * V, true, *reinterpret_cast<float(*)[V]>(w + e * V));
+    }
+    if (a.mu) {
+      load_v<float, V>(reinterpret_cast<const float*>(s.state + a.off_prev) + c + (size_t)s.flip * D, s.pos0 > 0, prev);
+      if constexpr (TAPS > 1) {
 #pragma unroll
-      for (int t = 0; t < MAX_TAPS; ++t) w[e][t] = t < taps ? a.w[(size_t)(c + e) * taps + t] : 0.f;
-#pragma unroll
-    for (int i = 0; i < MAX_MIX; ++i) load_v<float, V>(a.mu + (size_t)i * D + c, a.mu && i < a.n_mix, mu[i]);
+        for (int i = 0; i < MIX; ++i) load_v<float, V>(a.mu + (size_t)min(i, a.n_mix - 1) * D + c, true, mu[i]);
+      }
+    }
   }
   template <typename T>
   DEV void run(const JoinArgs& j, int row, int pos0, int c, const float (&h)[V]) {
     const ConvArgs& a = j.conv;
-    const int D = j.width, taps = a.taps;
+    const int D = j.width, taps = TAPS > 1 ? TAPS : a.taps;
     T* out = reinterpret_cast<T*>(a.out_t) + (size_t)row * a.ld + c;
     float y[V];
 #pragma unroll
     for (int e = 0; e < V; ++e) y[e] = 0.f;
-    if (small) {
+    if constexpr (TAPS > 1) {
 #pragma unroll
-      for (int t = 0; t < MAX_TAPS; ++t)
+      for (int t = 0; t < TAPS; ++t)
 #pragma unroll
-        for (int e = 0; e < V; ++e) y[e] += t < taps ? (t == taps - 1 ? h[e] : old[t < MAX_TAPS - 1 ? t : 0][e]) * w[e][t] : 0.f;
+        for (int e = 0; e < V; ++e) y[e] += (t == TAPS - 1 ? h[e] : old[t < KEPT ? t : 0][e]) * w[e * TAPS + t];
 #pragma unroll
-      for (int t = 1; t < MAX_TAPS - 1; ++t)
-        if (t < taps - 1) store_v<float, V>(next + (size_t)(t - 1) * D, old[t]);
+      for (int t = 1; t < KEPT; ++t) store_v<float, V>(next + (size_t)(t - 1) * D, old[t]);
     } else {
       for (int t = 0; t < taps - 1; ++t) {
         float o[V];
@@ -98,9 +97,9 @@ struct ConvOne {
       for (int e = 0; e < V; ++e) v[e] = y[e] + (prev[e] - y[e]) * m[e];
       store_v<T, V>(out + i * a.mix_stride, v);
     };
-    if (small) {
+    if constexpr (TAPS > 1) {
 #pragma unroll
-      for (int i = 0; i < MAX_MIX; ++i)
+      for (int i = 0; i < MIX; ++i)
         if (i < a.n_mix) blend(i, mu[i]);
     } else {
       for (int i = 0; i < a.n_mix; ++i) {
@@ -111,21 +110,32 @@ struct ConvOne {
     }
   }
 };
-// the sum of `parts` rows
-template <int V>
-DEV void load_sum(const float* p, bool in, int parts, size_t stride, float (&v)[V]) {
-  load_v<float, V>(p, in, v);
-  for (int k = 1; k < parts; k += 4) {
-    float q[4][V];
+// the sum of up to 8 rows, all requested at once (threads with many groups of elements: one row after the other)
+template <int V, bool MANY>
+struct LoadSum {
+  float q[MANY ? 1 : 8][V];
+  DEV void load(const float* p, bool in, int parts, size_t stride) {
+    if constexpr (MANY) {
+      load_v<float, V>(p, in, q[0]);
+#pragma unroll 1
+      for (int u = 1; u < parts; ++u) {
+        float w[V];
+        load_v<float, V>(p + u * stride, in, w);
 #pragma unroll
-    for (int u = 0; u < 4; ++u) load_v<float, V>(p + (k + u) * stride, in && k + u < parts, q[u]);
+        for (int e = 0; e < V; ++e) q[0][e] += w[e];
+      }
+    } else {
 #pragma unroll
-    for (int u = 0; u < 4; ++u)
-#pragma unroll
-      for (int e = 0; e < V; ++e) v[e] += q[u][e];
+      for (int u = 0; u < 8; ++u) load_v<float, V>(p + u * stride, in && u < max(parts, 1), q[u]);
+    }
   }
-}
-template <typename T, int NT, int VPT, int V, bool CONV>
+  DEV void sum(float (&v)[V]) const {
+#pragma unroll
+    for (int e = 0; e < V; ++e) v[e] = MANY ? q[0][e] : ((q[0][e] + q[1][e]) + (q[2][e] + q[3][e])) + ((q[4][e] + q[5][e]) + (q[6][e] + q[7][e]));
+  }
+};
+// CONV: taps of the convolution behind the norm (single tokens; ConvOne), 0: none
+template <typename T, int NT, int VPT, int V, int CONV>
 __global__ __launch_bounds__(NT) void join_kernel(const JoinArgs a) {
   __shared__ float red[NT / 64], s_w[64];
   __shared__ int s_pos[64];
@@ -134,17 +144,12 @@ __global__ __launch_bounds__(NT) void join_kernel(const JoinArgs a) {
   const int hrow = blockIdx.x;
   float x[VPT][V], add[VPT][V];
   auto at = [&](int i) { return V * (tid + i * NT); };
-  // with a convolution behind the norm: everything it reads, requested first (one group per thread) or together with its use (more)
-  ConvOne<V> cv;
+  // with a convolution behind the norm (single tokens: row = sequence): everything it reads and the norms' weights, requested behind the
+  // sum's operands (one group per thread) or together with its use (more)
+  ConvOne<V, (CONV > 1 ? CONV : 1)> cv;
   SeqDesc sq{};
-  float nw[V];
-  if constexpr (CONV) {
-    sq = a.p.seqs[a.p.row_seq[row]];
-    if constexpr (VPT == 1) {
-      cv.load(a, sq, at(0));
-      load_v<float, V>(a.norm_w + at(0), at(0) < D, nw);
-    }
-  }
+  float nw[V], pw[V];
+  if constexpr (CONV > 0) sq = a.p.seqs[row];
   if (a.y_t && tid < a.n_slots) {
     s_w[tid] = a.weight[(size_t)row * a.n_slots + tid];
     s_pos[tid] = a.slot_pos[(size_t)row * a.n_slots + tid];
@@ -156,16 +161,33 @@ __global__ __launch_bounds__(NT) void join_kernel(const JoinArgs a) {
 #pragma unroll
     for (int e = 0; e < V; ++e) add[i][e] = 0.f;
   }
+  if constexpr (CONV > 0 && VPT == 1) {
+    if (!a.mix_a) {
+      load_v<float, V>(a.norm_w + at(0), at(0) < D, nw);
+      cv.load(a, sq, at(0));
+    }
+  }
   if (a.mix_a) {
     const float* ma = a.mix_a + (size_t)row * a.mix_ld;
 #pragma unroll
-    for (int i = 0; i < VPT; ++i) load_sum<V>(ma + at(i), at(i) < D, a.parts_a, a.mix_stride, add[i]);
+    for (int i = 0; i < VPT; ++i) {
+      LoadSum<V, (VPT > 2)> q;
+      q.load(ma + at(i), at(i) < D, a.parts_a, a.mix_stride);
+      if constexpr (CONV > 0 && VPT == 1) {
+        if (a.post_w) load_v<float, V>(a.post_w + at(0), at(0) < D, pw);
+        load_v<float, V>(a.norm_w + at(0), at(0) < D, nw);
+        cv.load(a, sq, at(0));
+      }
+      q.sum(add[i]);
+    }
     if (a.mix_b) {
       const float* mb = a.mix_b + (size_t)row * a.mix_ld;
       float vb[VPT][V], sa = 0.f, sb = 0.f;
 #pragma unroll
       for (int i = 0; i < VPT; ++i) {
-        load_sum<V>(mb + at(i), at(i) < D, a.parts_b, a.mix_stride, vb[i]);
+        LoadSum<V, (VPT > 2)> q;
+        q.load(mb + at(i), at(i) < D, a.parts_b, a.mix_stride);
+        q.sum(vb[i]);
 #pragma unroll
         for (int e = 0; e < V; ++e) {
           sa += add[i][e] * add[i][e];
@@ -194,7 +216,12 @@ __global__ __launch_bounds__(NT) void join_kernel(const JoinArgs a) {
 #pragma unroll
       for (int i = 0; i < VPT; ++i) {
         float w[V];
-        load_v<float, V>(a.post_w + at(i), at(i) < D, w);
+        if constexpr (CONV > 0 && VPT == 1) {
+#pragma unroll
+          for (int e = 0; e < V; ++e) w[e] = pw[e];
+        } else {
+          load_v<float, V>(a.post_w + at(i), at(i) < D, w);
+        }
 #pragma unroll
         for (int e = 0; e < V; ++e) add[i][e] *= ra * (w[e] + a.norm_offset);
       }
@@ -233,21 +260,21 @@ __global__ __launch_bounds__(NT) void join_kernel(const JoinArgs a) {
   for (int i = 0; i < VPT; ++i) {
     if (at(i) >= D) continue;
     float w[V];
-    if constexpr (CONV && VPT == 1) {
+    if constexpr (CONV > 0 && VPT == 1) {
 #pragma unroll
       for (int e = 0; e < V; ++e) w[e] = nw[e];
     } else {
-      if constexpr (CONV) cv.load(a, sq, at(i));
+      if constexpr (CONV > 0) cv.load(a, sq, at(i));
       load_v<float, V>(a.norm_w + at(i), true, w);
     }
 #pragma unroll
     for (int e = 0; e < V; ++e) w[e] = x[i][e] * r * (w[e] + a.norm_offset);
-    if constexpr (CONV) cv.template run<T>(a, row, sq.pos0, at(i), w);
+    if constexpr (CONV > 0) cv.template run<T>(a, row, sq.pos0, at(i), w);
     else if (a.h_f) store_v<float, V>(a.h_f + (size_t)row * D + at(i), w);
     else store_v<T, V>(h + at(i), w);
   }
 }
-template <typename T, bool CONV>
+template <typename T, int CONV>
 static int join_t(hipStream_t st, const JoinArgs& a, int n) {
   const int D = a.width;
 #define JOIN(NT, VPT, V) hipLaunchKernelGGL((join_kernel<T, NT, VPT, V, CONV>), dim3(n), dim3(NT), 0, st, a)
@@ -267,8 +294,9 @@ static int join_t(hipStream_t st, const JoinArgs& a, int n) {
 int launch_join(hipStream_t st, const JoinArgs& a, bool f32) {
   const int n = a.only_want ? a.p.n_want : a.p.rows;
   if (n < 1) DSK_FAIL(DSK_ERR_INVALID, "join: no rows");
-  if (a.conv.w) return f32 ? join_t<float, true>(st, a, n) : join_t<bf16, true>(st, a, n);
-  return f32 ? join_t<float, false>(st, a, n) : join_t<bf16, false>(st, a, n);
+  if (!a.conv.w) return f32 ? join_t<float, 0>(st, a, n) : join_t<bf16, 0>(st, a, n);
+  if (a.conv.taps == 4 && a.conv.n_mix <= ConvOne<1, 4>::MAX_MIX) return f32 ? join_t<float, 4>(st, a, n) : join_t<bf16, 4>(st, a, n);
+  return f32 ? join_t<float, 1>(st, a, n) : join_t<bf16, 1>(st, a, n);
 }
 
 // ---- convolution in front of a sublayer, portions --------------------------------------------------------

@@ -40,7 +40,7 @@ template <typename T>
 __global__ __launch_bounds__(PREP_NT) void latent_prep_kernel(const LatentArgs a) {
   constexpr int NT = PREP_NT, U = 4;  // U elements of either latent per thread wait in registers; larger ones are read again
   __shared__ float red[2 * NT / 64];
-  const int row = blockIdx.x, tid = threadIdx.x, half = a.rot_dims >> 1, ld = a.rank_p + a.rot_p;
+  const int row = blockIdx.x, tid = threadIdx.x, half = a.rot_dims >> 1, ld = a.rank_p + a.rot_p, cq_k = (a.q_rank + 63) & ~63;
   const SeqDesc s = a.p.seqs[a.p.row_seq[row]];
   const int pos = s.pos0 + row - s.row0;
   const float *q = a.proj_f + (size_t)row * a.ld + a.col_q, *kv = a.proj_f + (size_t)row * a.ld + a.col_kv;
@@ -86,10 +86,10 @@ __global__ __launch_bounds__(PREP_NT) void latent_prep_kernel(const LatentArgs a
 #pragma unroll
   for (int u = 0; u < U; ++u) {
     const int i = tid + u * NT;
-    if (i < a.cq_ld) cq[i] = (T)(xq[u] * rq * wq[u]);
+    if (i < cq_k) cq[i] = (T)(xq[u] * rq * wq[u]);
     if (i < a.rank_p) lat[i] = (T)(xk[u] * rk * wk[u]);
   }
-  for (int i = tid + U * NT; i < a.cq_ld; i += NT) cq[i] = (T)(i < a.q_rank ? q[i] * rq * a.q_norm[i] : 0.f);
+  for (int i = tid + U * NT; i < cq_k; i += NT) cq[i] = (T)(i < a.q_rank ? q[i] * rq * a.q_norm[i] : 0.f);
   for (int i = tid + U * NT; i < a.rank_p; i += NT) lat[i] = (T)(i < a.kv_rank ? kv[i] * rk * a.kv_norm[i] : 0.f);
   for (int j = tid; j < a.rot_p; j += NT) lat[a.rank_p + j] = (T)(j < a.rot_dim ? turned([&](int i) { return kv[a.kv_rank + i]; }, turn, a.rot_dims, j) : 0.f);
 }
@@ -187,6 +187,16 @@ __global__ __launch_bounds__(FEW_NT) void latent_few_kernel(const LatentArgs a) 
   T* pw = reinterpret_cast<T*>(red + FEW_NW * 64);        // [16][LP] weights
   const T* ring = reinterpret_cast<const T*>(s.state + a.off_c);
   const int ng = ld >> 3, first = pos - seen + 1 + k0;
+  // the query operands of a wave's part, ahead of everything else (the first ones; larger latents read the rest as they go)
+  constexpr int QA = sizeof(T) == 2 ? 8 : 4;
+  const int kt16 = wave % KTILES, part = wave / KTILES, kts = a.rank_p >> 5;
+  frag qf[QA];
+  auto query = [&](int h0) { return reinterpret_cast<const T*>(a.qa_t) + ((size_t)i * a.heads + min(h0 + c16, a.heads - 1)) * a.rank_p + g * 8; };
+  auto ahead = [&](int h0) {
+#pragma unroll
+    for (int u = 0; u < QA; ++u) qf[u] = *reinterpret_cast<const frag*>(query(h0) + min(part + u * PARTS, kts - 1) * 32);
+  };
+  ahead(0);
   constexpr int IN_FLIGHT = sizeof(T) == 2 ? 12 : 6;
   for (int u0 = tid; u0 < N * ng; u0 += FEW_NT * IN_FLIGHT) {
     frag f[IN_FLIGHT];
@@ -212,15 +222,14 @@ __global__ __launch_bounds__(FEW_NT) void latent_few_kernel(const LatentArgs a) 
     }
     __syncthreads();
     {
-      const int kt16 = wave % KTILES, part = wave / KTILES;
-      const T* qa = reinterpret_cast<const T*>(a.qa_t) + ((size_t)i * a.heads + min(h0 + c16, a.heads - 1)) * a.rank_p + g * 8;
       f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-      for (int kt = part; kt < ld >> 5; kt += PARTS) {
-        const frag k = *reinterpret_cast<const frag*>(lat + (size_t)(kt16 * 16 + c16) * LD + kt * 32 + g * 8);
-        const frag q = kt * 32 < a.rank_p ? *reinterpret_cast<const frag*>(qa + kt * 32) : *reinterpret_cast<const frag*>(qr + c16 * LQ + kt * 32 - a.rank_p + g * 8);
-        acc = mma(k, q, acc);
-      }
+      auto score = [&](int kt, const frag& q) { acc = mma(*reinterpret_cast<const frag*>(lat + (size_t)(kt16 * 16 + c16) * LD + kt * 32 + g * 8), q, acc); };
+#pragma unroll
+      for (int u = 0; u < QA; ++u)
+        if (part + u * PARTS < kts) score(part + u * PARTS, qf[u]);
+      for (int kt = part + QA * PARTS; kt < kts; kt += PARTS) score(kt, *reinterpret_cast<const frag*>(query(h0) + kt * 32));
+      for (int kt = part; kt < a.rot_p >> 5; kt += PARTS) score(kts + kt, *reinterpret_cast<const frag*>(qr + c16 * LQ + kt * 32 + g * 8));
+      if (h0 + 16 < a.heads) ahead(h0 + 16);
       red[(part * KTILES + kt16) * 64 + lane] = acc;
     }
     __syncthreads();

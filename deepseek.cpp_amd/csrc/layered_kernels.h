@@ -250,7 +250,7 @@ struct LatentArgs {
   const float* proj_f;      // 32-bit projections [rows][ld]: query latent, then [latent, rotated key part]
   int ld, col_q, col_kv;
   const float *q_norm, *kv_norm, *freq;
-  void* cq_t;               // normed query latents [rows][cq_ld]
+  void* cq_t;               // normed query latents [rows][cq_ld], zero up to a multiple of 64 columns
   int cq_ld;
   float* turn;              // cosines, then sines of a row's angles [rows][rot_dims]
   const void* q_t;          // queries [rows][q_ld], per head [dim_p][rot_p], not rotated yet

@@ -114,7 +114,7 @@ struct LayeredModel : ModelHead {
   // sandwich layers, latent attention
   float *h_f = nullptr, *turn = nullptr, *lat_part = nullptr, *lat_ml = nullptr;
   char *cq = nullptr, *lq = nullptr, *lat = nullptr, *kv = nullptr, *qabs = nullptr;
-  int mixes = 1, lq_ld = 0, max_window = 0, key_cap = 0;  // mixes: blends of h; key_cap: rows of the key workspace
+  int mixes = 1, lq_ld = 0, cq_ld = 0, kv_ld = 0, max_window = 0, key_cap = 0;  // mixes: blends of h; key_cap: rows of the key workspace
   float *weight = nullptr, *logits = nullptr, *trace_x = nullptr, *sample_scratch = nullptr;
   int *slot_pos = nullptr, *chosen = nullptr, *count = nullptr, *cursor = nullptr, *slot_row = nullptr, *tiles = nullptr, *n_tiles = nullptr, *active = nullptr,
       *active_slot = nullptr, *n_active = nullptr, *next_dev = nullptr;
@@ -581,6 +581,8 @@ int alloc_work(LayeredModel* m) {
   m->h_ld = (int)up(D, 64);
   m->mix_ld = m->y_ld = (int)up(D, 16);
   m->out_ld = std::max(out, 64);
+  m->cq_ld = (int)cq;
+  m->kv_ld = (int)kv;
   m->low_ld = low;
   m->slots = tmax;
   m->ld_logits = m->head.rt * 16;
@@ -590,10 +592,10 @@ int alloc_work(LayeredModel* m) {
   if (m->max_window) {
     m->key_cap = m->piece + m->max_window;
     DSK_TRY(dev_alloc_n(m, &m->turn, n * turn));
-    DSK_TRY(dev_alloc(m, (void**)&m->cq, n * cq * e));
+    DSK_TRY(dev_alloc(m, (void**)&m->cq, n * m->cq_ld * e));
     DSK_TRY(dev_alloc(m, (void**)&m->lq, n * m->lq_ld * e));
     DSK_TRY(dev_alloc(m, (void**)&m->lat, m->key_cap * key * e));
-    DSK_TRY(dev_alloc(m, (void**)&m->kv, m->key_cap * kv * e));
+    DSK_TRY(dev_alloc(m, (void**)&m->kv, m->key_cap * m->kv_ld * e));
     DSK_TRY(dev_alloc(m, (void**)&m->qabs, FEW * qabs * e));
     DSK_TRY(dev_alloc_n(m, &m->lat_part, lat_part));
     DSK_TRY(dev_alloc_n(m, &m->lat_ml, lat_ml));
@@ -752,7 +754,7 @@ ChunkAttnArgs attn_args(LayeredModel* m, const PassDesc& p, const LayerSpec& l, 
   a.off_k = w.off_k;
   a.off_v = w.off_v;
   a.out_t = m->out_a;
-  a.out_ld = w.a_o.kt * 32;
+  a.out_ld = m->out_ld;
   return a;
 }
 int attention(LayeredModel* m, const ChunkAttnArgs& a) {
@@ -790,7 +792,7 @@ MlstmArgs mlstm_args(LayeredModel* m, const PassDesc& p, const LayerSpec& l, con
   a.off_n = w.off_mn;
   a.off_m = w.off_mm;
   a.out_t = out;
-  a.out_ld = w.m_o.kt * 32;
+  a.out_ld = m->out_ld;
   return a;
 }
 // a pass of few, long sequences runs its recurrences over chunks of 16 tokens; many short ones go token by token
@@ -840,7 +842,7 @@ DeltaArgs delta_args(LayeredModel* m, const PassDesc& p, const LayerSpec& l, con
   a.off_s = w.off_ds;
   a.off_conv = w.off_dc;
   a.out_t = m->out_a;
-  a.out_ld = w.d_o.kt * 32;
+  a.out_ld = m->out_ld;
   return a;
 }
 int delta(LayeredModel* m, const DeltaArgs& a, const LayerW& w, bool few) {
@@ -910,7 +912,7 @@ WkvArgs wkv_args(LayeredModel* m, const PassDesc& p, const LayerSpec& l, const L
   a.o = m->o;
   a.off_s = w.off_ws;
   a.out_t = m->out_a;
-  a.out_ld = w.w_o.kt * 32;
+  a.out_ld = m->out_ld;
   return a;
 }
 int wkv(LayeredModel* m, const WkvArgs& a, const LayerW& w, bool few) {
@@ -948,16 +950,16 @@ LatentArgs latent_args(LayeredModel* m, const PassDesc& p, const LayerSpec& l, c
   a.kv_norm = w.l_kvn;
   a.freq = w.freq;
   a.cq_t = m->cq;
-  a.cq_ld = w.l_uq.kt * 32;
+  a.cq_ld = m->cq_ld;
   a.turn = m->turn;
   a.q_t = m->lq;
   a.q_ld = m->lq_ld;
   a.lat_t = m->lat;
   a.kv_t = m->kv;
-  a.kv_ld = w.l_ukv.rt * 16;
+  a.kv_ld = m->kv_ld;
   a.off_c = w.off_lc;
   a.out_t = m->out_a;
-  a.out_ld = w.l_o.kt * 32;
+  a.out_ld = m->out_ld;
   a.splits = std::min(m->splits, latent_splits(m, s));
   a.qa_t = m->qabs;
   a.part = m->lat_part;
@@ -1052,22 +1054,22 @@ int run_layer(LayeredModel* m, const PassDesc& p, int l, bool few) {
   MixFewArgs f{};
   if (s.has_attn) {
     f.attn = attn_args(m, p, s, w);
-    outs[n_out++] = mix_lin(m, w.a_o, m->out_a, w.a_o.kt * 32, p.rows, few);
+    outs[n_out++] = mix_lin(m, w.a_o, m->out_a, m->out_ld, p.rows, few);
   }
   if (s.has_mlstm) {
     f.mlstm = mlstm_args(m, p, s, w, n_out ? m->out_b : m->out_a);
-    outs[n_out] = mix_lin(m, w.m_o, n_out ? m->out_b : m->out_a, w.m_o.kt * 32, p.rows, few, n_out > 0);
+    outs[n_out] = mix_lin(m, w.m_o, n_out ? m->out_b : m->out_a, m->out_ld, p.rows, few, n_out > 0);
     ++n_out;
   }
   if (s.has_delta) {
     f.delta = delta_args(m, p, s, w);
-    outs[n_out++] = mix_lin(m, w.d_o, m->out_a, w.d_o.kt * 32, p.rows, few);
+    outs[n_out++] = mix_lin(m, w.d_o, m->out_a, m->out_ld, p.rows, few);
   }
   if (s.has_wkv) {
     f.wkv = wkv_args(m, p, s, w);
-    outs[n_out++] = mix_lin(m, w.w_o, m->out_a, w.w_o.kt * 32, p.rows, few);
+    outs[n_out++] = mix_lin(m, w.w_o, m->out_a, m->out_ld, p.rows, few);
   }
-  if (s.has_latent) outs[n_out++] = mix_lin(m, w.l_o, m->out_a, w.l_o.kt * 32, p.rows, few);
+  if (s.has_latent) outs[n_out++] = mix_lin(m, w.l_o, m->out_a, m->out_ld, p.rows, few);
   const MoeArgs e = s.has_moe ? moe_args(m, p, s, w) : MoeArgs{};
   f.rows = p.rows;
   f.has_attn = s.has_attn;

@@ -2,6 +2,7 @@
 //
 //   lin_kernel      prompts: 128 features x 128 rows per workgroup, 4 waves of 64 x 64, both operands through LDS in fragment
 //                   order (global_load_lds, 16 bytes per lane: LDS reads are lane-linear, no bank conflicts), two buffers
+//   lin_big_kernel  the same with 256 x 256 and a ring of four stages, where there are enough of such tiles (bf16)
 //   few_kernel      up to 16 rows (decoding): 4 waves share 16 features and split k; weights stream from HBM straight into the
 //                   MFMA operand registers, 1 KiB contiguous per wave and load
 // Both take plain products and the experts' (rows gathered per expert); a launch of few_kernel can hold several products.
@@ -102,8 +103,15 @@ DEV void store_glu(const LinArgs& a, int row, int feature, const f32x4& g, const
   *reinterpret_cast<four*>(reinterpret_cast<T*>(a.out_t) + (size_t)row * a.ld_t + feature) = to_four<T>(v);
 }
 
-// k tiles per part: even, so that a part is whole steps of the prompt kernel
-__host__ DEV int part_tiles(const LinArgs& a) { return a.parts > 1 ? ((a.kt / 2 + a.parts - 1) / a.parts) * 2 : a.kt; }
+// Workgroups go round robin over the 8 XCDs, each with an L2 of its own: XCD x takes the x-th eighth of the tiles, in order, so that the
+// tiles of one weight tile (and then its neighbours) meet in one L2.
+DEV int xcd_range(int b, int n) {
+  const int x = b & 7, base = n >> 3, extra = n & 7;
+  return x * base + min(x, extra) + (b >> 3);
+}
+// k tiles per part: even, so that a part is whole steps of the prompt kernels
+__host__ DEV int part_tiles(int kt, int parts) { return parts > 1 ? ((kt / 2 + parts - 1) / parts) * 2 : kt; }
+__host__ DEV int part_tiles(const LinArgs& a) { return part_tiles(a.kt, a.parts); }
 // the operand a product's features from `feature` on read
 template <typename T>
 DEV const T* operand(const LinArgs& a, int feature) {
@@ -114,6 +122,10 @@ DEV const T* operand(const LinArgs& a, int feature) {
 // ---- prompts -------------------------------------------------------------------------------------
 // grid.x: row tiles of 128 (experts: entries of the tile table), grid.y: feature tiles of 128.
 // rows: a gather table (slot -> row) or nullptr; out rows are row0 + local row.
+// A block of activations (16 rows x 32 columns, bf16) arrives row by row, four lanes to the 64 bytes of a row; inside a row the groups of 8
+// columns are exchanged by the row's place so that the lanes that read one group of 16 rows meet every LDS bank once.
+DEV int block_group(int lane) { return (lane & 3) ^ (lane >> 4); }                                  // the group lane l of a load brings
+DEV int block_at(int lane) { return ((lane & 15) * 4 + ((lane >> 4) ^ ((lane >> 2) & 3))) * 16; }  // where lane l of an operand reads
 template <typename T>
 DEV void lin_body(const LinArgs& a, const int* gather, int row0, int n_rows, int f0, int k0, int k1, char* lds) {
   typedef typename Frag<T>::type frag;
@@ -130,9 +142,9 @@ DEV void lin_body(const LinArgs& a, const int* gather, int row0, int n_rows, int
     const int t = 2 * wave + i;
     const int rt = min(rt0 + t, a.rt - 1);  // (tiles past the end: any valid one, never stored)
     src_w[i] = reinterpret_cast<const char*>(a.w) + (size_t)rt * a.kt * 1024 + lane * 16;
-    int r = min(t * 16 + (lane & 15), n_rows - 1);
+    int r = min(t * 16 + (sizeof(T) == 2 ? lane >> 2 : lane & 15), n_rows - 1);
     r = gather ? gather[row0 + r] : row0 + r;
-    src_a[i] = operand<T>(a, f0) + (size_t)r * a.lda + (lane >> 4) * 8;
+    src_a[i] = operand<T>(a, f0) + (size_t)r * a.lda + (sizeof(T) == 2 ? block_group(lane) : lane >> 4) * 8;
   }
   auto stage = [&](int kt, char* buf) {
 #pragma unroll
@@ -150,7 +162,7 @@ DEV void lin_body(const LinArgs& a, const int* gather, int row0, int n_rows, int
   auto read_a = [&](const char* buf, int slot) {
     frag f;
     if constexpr (sizeof(T) == 2) {
-      f = *reinterpret_cast<const frag*>(buf + 16 * 1024 + slot * AB + lane * 16);
+      f = *reinterpret_cast<const frag*>(buf + 16 * 1024 + slot * AB + block_at(lane));
     } else {
       const f32x4 lo = *reinterpret_cast<const f32x4*>(buf + 16 * 1024 + slot * AB + lane * 16);
       const f32x4 hi = *reinterpret_cast<const f32x4*>(buf + 16 * 1024 + slot * AB + 1024 + lane * 16);
@@ -200,11 +212,95 @@ DEV void lin_body(const LinArgs& a, const int* gather, int row0, int n_rows, int
   }
 }
 template <typename T>
-__global__ __launch_bounds__(256) void lin_kernel(LinArgs a) {
+__global__ __launch_bounds__(256) void lin_kernel(LinArgs a, const int row_tiles, const int tiles) {
   extern __shared__ __attribute__((aligned(16))) char lds[];
-  const int row0 = blockIdx.x * 128, per = part_tiles(a), k0 = blockIdx.z * per;
-  a.out_f += blockIdx.z * a.part_stride;
-  lin_body<T>(a, nullptr, row0, min(128, a.rows - row0), blockIdx.y * 128, k0, min(a.kt, k0 + per), lds);
+  const int b = xcd_range(blockIdx.x, tiles), row0 = b % row_tiles * 128, per = part_tiles(a), k0 = blockIdx.y * per;
+  a.out_f += blockIdx.y * a.part_stride;
+  lin_body<T>(a, nullptr, row0, min(128, a.rows - row0), b / row_tiles * 128, k0, min(a.kt, k0 + per), lds);
+}
+
+// 256 features x 256 rows per workgroup: 8 waves of 128 x 64; twice the matrix work per byte staged.  A ring of RING stages of one k tile
+// (32 KiB): while a tile is multiplied the next one's operands are read into the other set of registers, and RING - 1 more are on their way.
+enum { RING = 4 };
+__global__ __launch_bounds__(512) __attribute__((amdgpu_waves_per_eu(2, 2))) void lin_big_kernel(LinArgs a, const int row_tiles, const int tiles) {
+  extern __shared__ __attribute__((aligned(16))) char lds[];
+  constexpr int STAGE = 32 * 1024;
+  const int b = xcd_range(blockIdx.x, tiles), row0 = b % row_tiles * 256, f0 = b / row_tiles * 256, per = part_tiles(a), k0 = blockIdx.y * per, n = min(a.kt - k0, per);
+  a.out_f += blockIdx.y * a.part_stride;
+  const int n_rows = min(256, a.rows - row0);
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int wm = wave & 1, wn = wave >> 1, rt0 = f0 >> 4;
+  const char *src_w[2], *src_a[2];  // this wave's share of a stage: weight tiles and row groups 2 * wave + {0, 1}
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const int t = 2 * wave + i;
+    src_w[i] = reinterpret_cast<const char*>(a.w) + ((size_t)min(rt0 + t, a.rt - 1) * a.kt + k0) * 1024 + lane * 16;
+    src_a[i] = reinterpret_cast<const char*>(operand<bf16>(a, f0) + (size_t)(row0 + min(t * 16 + (lane >> 2), n_rows - 1)) * a.lda + (size_t)k0 * 32 + block_group(lane) * 8);
+  }
+  auto stage = [&](int kt, char* buf) {  // (past the end: the last tile again, never read)
+    kt = min(kt, n - 1);
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const int slot = 2 * wave + i;
+      __builtin_amdgcn_global_load_lds((gptr)(src_w[i] + (size_t)kt * 1024), (lptr)(buf + slot * 1024), 16, 0, 0);
+      __builtin_amdgcn_global_load_lds((gptr)(src_a[i] + (size_t)kt * 64), (lptr)(buf + 16 * 1024 + slot * 1024), 16, 0, 0);
+    }
+  };
+  f32x4 acc[8][4];
+#pragma unroll
+  for (int i = 0; i < 8; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+  struct Operands {
+    bf16x8 w[8], x[4];
+  };
+  auto read = [&](const char* buf, Operands& o) {
+#pragma unroll
+    for (int j = 0; j < 4; ++j) o.x[j] = *reinterpret_cast<const bf16x8*>(buf + 16 * 1024 + (wn * 4 + j) * 1024 + block_at(lane));
+#pragma unroll
+    for (int i = 0; i < 8; ++i) o.w[i] = *reinterpret_cast<const bf16x8*>(buf + (wm * 8 + i) * 1024 + lane * 16);
+  };
+  int cur = 0;
+  auto step = [&](int kt, const Operands& now, Operands& next) {
+    // tile kt + 1 is here when at most the loads of RING - 2 tiles are outstanding; behind the barrier everybody's are, and everybody holds
+    // tile kt in registers, so that its buffer takes tile kt + RING
+    asm volatile("s_waitcnt vmcnt(%0)" ::"n"(4 * (RING - 2)) : "memory");
+    lds_barrier();
+    stage(kt + RING, lds + cur * STAGE);
+    cur = cur + 1 == RING ? 0 : cur + 1;
+    read(lds + cur * STAGE, next);
+#pragma unroll
+    for (int i = 0; i < 8; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) acc[i][j] = mma(now.w[i], now.x[j], acc[i][j]);
+#pragma unroll
+    for (int i = 0; i < 12; ++i) {  // one LDS read, then matrix work that does not wait for it
+      __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
+      __builtin_amdgcn_sched_group_barrier(0x008, 2, 0);
+    }
+    __builtin_amdgcn_sched_group_barrier(0x008, 8, 0);
+  };
+  Operands p, q;
+#pragma unroll
+  for (int i = 0; i < RING; ++i) stage(i, lds + i * STAGE);
+  asm volatile("s_waitcnt vmcnt(%0)" ::"n"(4 * (RING - 1)) : "memory");
+  lds_barrier();
+  read(lds, p);
+  for (int kt = 0; kt < n; kt += 2) {  // (n is even)
+    step(kt, p, q);
+    step(kt + 1, q, p);
+  }
+  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const int r = wn * 64 + j * 16 + (lane & 15);
+    if (r >= n_rows) continue;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      const int rt = rt0 + wm * 8 + i;
+      if (rt < a.rt) store_plain<bf16>(a, row0 + r, rt * 16 + (lane >> 4) * 4, acc[i][j]);
+    }
+  }
 }
 
 static LinArgs expert_lin(const MoeArgs& m, bool down) {  // the parts of an expert product that do not depend on the expert
@@ -333,17 +429,51 @@ static int allow_lds(K k, int bytes) {
   HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize, bytes));
   return DSK_OK;
 }
+// Microseconds a prompt product takes on 256 compute units, by measurement: two workgroups of 128 x 128 on one work 1.3 us on a step of 64
+// columns (one alone 1.05), one of 256 x 256 takes 1.84 us and starts and ends slower; a part more writes and reads its sums.
+static double lin_cost(int rows, int rt, int kt, int parts, bool big) {
+  const double k = part_tiles(kt, parts) / 2, sums = (parts - 1) * 3.2e-5 * rows * rt;
+  if (big) return cdiv(cdiv(rows, 256) * cdiv(rt, 16) * parts, 256) * (15 + 1.84 * k) + sums;
+  const int n = cdiv(rows, 128) * cdiv(rt, 8) * parts;
+  return (n <= 256 ? 1.05 * k : cdiv(n, 512) * 1.3 * k) + 5 + sums;
+}
+static bool lin_big(int rows, int rt, int kt, int parts, int a_seg, bool f32) {
+  return !f32 && !(a_seg & 255) && lin_cost(rows, rt, kt, parts, true) < lin_cost(rows, rt, kt, parts, false);
+}
+int lin_parts(int rows, int rt, int kt, bool f32, int most) {
+  int best = 1;
+  double least = 0;
+  for (int n = 1; n <= most && (n == 1 || kt / n >= 16); ++n) {
+    const double c = std::min(lin_cost(rows, rt, kt, n, false), f32 ? 1e9 : lin_cost(rows, rt, kt, n, true));
+    if (n == 1 || c < least) {
+      least = c;
+      best = n;
+    }
+  }
+  return cdiv(kt, part_tiles(kt, best));  // (no part may be empty)
+}
+int lin_parts_few(int rt, int kt, int most) {
+  const int n = std::max(std::min({1024 / rt, kt / 16, most}), 1);
+  return cdiv(kt, part_tiles(kt, n));
+}
 int launch_lin(hipStream_t st, const LinArgs& a, bool f32) {
   DSK_TRY(check_lin(a, "lin"));
   if ((a.a_seg & 127) || a.row_seq) DSK_FAIL(DSK_ERR_INVALID, "lin: %d features per operand", a.a_seg);
-  const dim3 grid(cdiv(a.rows, 128), cdiv(a.rt, 8), std::max(a.parts, 1));
+  if (lin_big(a.rows, a.rt, a.kt, std::max(a.parts, 1), a.a_seg, f32)) {
+    const int row_tiles = cdiv(a.rows, 256), tiles = row_tiles * cdiv(a.rt, 16);
+    DSK_TRY(allow_lds(lin_big_kernel, RING * 32 * 1024));
+    hipLaunchKernelGGL(lin_big_kernel, dim3(tiles, std::max(a.parts, 1)), dim3(512), RING * 32 * 1024, st, a, row_tiles, tiles);
+    return DSK_OK;
+  }
+  const int row_tiles = cdiv(a.rows, 128), tiles = row_tiles * cdiv(a.rt, 8);
+  const dim3 grid(tiles, std::max(a.parts, 1));
   const int lds = lin_lds(f32);
   if (f32) {
     DSK_TRY(allow_lds(lin_kernel<float>, lds));
-    hipLaunchKernelGGL(lin_kernel<float>, grid, dim3(256), lds, st, a);
+    hipLaunchKernelGGL(lin_kernel<float>, grid, dim3(256), lds, st, a, row_tiles, tiles);
   } else {
     DSK_TRY(allow_lds(lin_kernel<bf16>, lds));
-    hipLaunchKernelGGL(lin_kernel<bf16>, grid, dim3(256), lds, st, a);
+    hipLaunchKernelGGL(lin_kernel<bf16>, grid, dim3(256), lds, st, a, row_tiles, tiles);
   }
   return DSK_OK;
 }

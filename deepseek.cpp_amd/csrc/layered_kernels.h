@@ -62,6 +62,9 @@ struct LinArgs {
   const int* row_seq;     // launch_lin_few: output row i reads the first row of sequence row_seq[i] of seqs (nullptr: row i)
   const SeqDesc* seqs;
 };
+// parts worth splitting k into, at most `most`: launch_lin, launch_lin_few
+int lin_parts(int rows, int rt, int kt, bool f32, int most);
+int lin_parts_few(int rt, int kt, int most);
 int launch_lin(hipStream_t st, const LinArgs& a, bool f32);          // any number of rows (tiles of 128)
 int launch_lin_few(hipStream_t st, const LinArgs* a, int n, bool f32);  // up to 16 rows; n <= 4 products in one launch
 

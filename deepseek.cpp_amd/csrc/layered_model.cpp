@@ -676,11 +676,8 @@ LinArgs lin_f(const PackedMat& w, const void* a, int lda, int rows, float* out, 
 }
 // A product whose output the next residual sum reads (mix_a; second: mix_b), split over k where its tiles alone leave compute units idle
 LinArgs mix_lin(LayeredModel* m, const PackedMat& w, const void* a, int lda, int rows, bool few, bool second = false) {
-  const int tiles = few ? w.rt : ((rows + 127) / 128) * ((w.rt + 7) / 8);
-  const int n = std::max(std::min({few ? 1024 / tiles : 512 / tiles, w.kt / 16, (int)(few ? MIX_PARTS_FEW : MIX_PARTS)}), 1);
-  const int per = (w.kt / 2 + n - 1) / n * 2;  // (no part may be empty)
   LinArgs l = lin_f(w, a, lda, rows, second ? m->mix_b : m->mix_a, m->mix_ld);
-  l.parts = m->mix_parts[second] = (w.kt + per - 1) / per;
+  l.parts = m->mix_parts[second] = few ? lin_parts_few(w.rt, w.kt, MIX_PARTS_FEW) : lin_parts(rows, w.rt, w.kt, m->f32, MIX_PARTS);
   l.part_stride = m->mix_stride = (size_t)rows * m->mix_ld;
   return l;
 }

@@ -83,7 +83,7 @@ struct ChunkKeys {
   }
 };
 template <typename T, int KT, int VTL>
-__global__ __launch_bounds__(256) void chunk_attn_kernel(const ChunkAttnArgs a) {
+ATTN_KERNEL(T) void chunk_attn_kernel(const ChunkAttnArgs a) {
   const int h = blockIdx.y, tile = gridDim.x - 1 - blockIdx.x;  // (a sequence's last tiles have the most keys: they start first)
   const SeqDesc s = a.p.seqs[a.p.qtile[2 * tile]];
   attn_tile<T, KT, VTL>(ChunkKeys<T>{a, s, h, h / (a.heads / a.kv_heads)}, s, a.p.qtile[2 * tile + 1], a.dim_p >> 5, a.vdim_p >> 4, a.vdim, a.scale,
@@ -114,21 +114,17 @@ int launch_chunk_prep(hipStream_t st, const ChunkAttnArgs& a, bool f32) {
   else hipLaunchKernelGGL(chunk_prep_kernel<bf16>, grid, dim3(256), 0, st, a);
   return DSK_OK;
 }
-template <typename T, int KT, int VTL>
-static int attn_t(hipStream_t st, const ChunkAttnArgs& a) {
-  const size_t lds = attn_tile_lds<T>(a.dim_p, a.vdim_p);
-  auto k = chunk_attn_kernel<T, KT, VTL>;
-  HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
-  hipLaunchKernelGGL(k, dim3(a.p.n_qtiles, a.heads), dim3(256), lds, st, a);
-  return DSK_OK;
-}
 template <typename T>
-static int attn_dims(hipStream_t st, const ChunkAttnArgs& a) {
-  if (a.dim_p <= 128 && a.vdim_p <= 128) return attn_t<T, 4, 8>(st, a);
-  if (a.dim_p <= 256 && a.vdim_p <= 256) return attn_t<T, 8, 16>(st, a);
-  DSK_FAIL(DSK_ERR_UNSUPPORTED, "chunk attention: key size %d, value size %d (max 256)", a.dim, a.vdim);
+static int attn_t(hipStream_t st, const ChunkAttnArgs& a) {
+  return attn_sizes(a.dim_p >> 5, a.vdim_p >> 4, [&](auto kt, auto vt) -> int {
+    constexpr int KT = decltype(kt)::value, VTL = decltype(vt)::value, lds = attn_tile_lds<T, KT, VTL>();
+    auto k = chunk_attn_kernel<T, KT, VTL>;
+    HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize, lds));
+    hipLaunchKernelGGL(k, dim3(a.p.n_qtiles, a.heads), dim3(256), lds, st, a);
+    return (int)DSK_OK;
+  }, "chunk attention");
 }
-int launch_chunk_attn(hipStream_t st, const ChunkAttnArgs& a, bool f32) { return f32 ? attn_dims<float>(st, a) : attn_dims<bf16>(st, a); }
+int launch_chunk_attn(hipStream_t st, const ChunkAttnArgs& a, bool f32) { return f32 ? attn_t<float>(st, a) : attn_t<bf16>(st, a); }
 int launch_chunk_store(hipStream_t st, const ChunkAttnArgs& a, bool f32) {
   if (f32) hipLaunchKernelGGL(chunk_store_kernel<float>, dim3(a.p.rows), dim3(256), 0, st, a);
   else hipLaunchKernelGGL(chunk_store_kernel<bf16>, dim3(a.p.rows), dim3(256), 0, st, a);

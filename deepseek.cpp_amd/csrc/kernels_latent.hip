@@ -5,6 +5,7 @@
 //   latent_prep     norms of the query latent and of c, the angles' cosines and sines, the rotated key part
 //   latent_gather   the older rows that a portion of several tokens sees, from the ring, in front of the portion's rows; one matrix product
 //                   then expands them all to keys and values per head
+//   latent_turn     the rotation of the queries
 //   latent_attn     64 queries per workgroup (attn_tile.h): a key is its head's expanded part, then the shared rotated one
 //   latent_store    the portion's last rows into the ring (behind the attention's gather)
 //   latent_few      single tokens: the query comes carried into the latent space (W_uk^T q), so a score is one product with a ring row and
@@ -122,6 +123,23 @@ __global__ __launch_bounds__(256) void latent_store_kernel(const LatentArgs a) {
   for (int e = (threadIdx.x & 63) * 8; e < ld; e += 512) *reinterpret_cast<frag*>(dst + e) = *reinterpret_cast<const frag*>(src + e);
 }
 
+// ---- rotation of the queries, in place (portions of several tokens; latent_few rotates its own) -----------------------
+template <typename T>
+__global__ __launch_bounds__(256) void latent_turn_kernel(const LatentArgs a) {
+  const int row = blockIdx.x, half = a.rot_dims >> 1, hd = a.dim_p + a.rot_p;
+  if (a.p.seqs[a.p.row_seq[row]].len == 1) return;
+  const float* turn = a.turn + (size_t)row * a.rot_dims;
+  T* q = reinterpret_cast<T*>(a.q_t) + (size_t)row * a.q_ld + a.dim_p;
+#pragma unroll 4
+  for (int i = threadIdx.x; i < a.heads * half; i += 256) {
+    const int j = i % half;
+    T* p = q + (size_t)(i / half) * hd + j;
+    const float u = (float)p[0], v = (float)p[half], c = turn[j], s = turn[half + j];
+    p[0] = (T)(u * c - v * s);
+    p[half] = (T)(v * c + u * s);
+  }
+}
+
 // ---- portions of several tokens --------------------------------------------------------------------------------------
 template <typename T>
 struct LatentKeys {
@@ -133,16 +151,7 @@ struct LatentKeys {
   DEV int first(int pos) const { return max(0, pos - a.window + 1); }
   DEV size_t key_row(int pos) const { return (size_t)(s.key0 + s.hist + pos - s.pos0); }
   DEV frag q(int row, int gr) const {
-    const T* p = reinterpret_cast<const T*>(a.q_t) + (size_t)(s.row0 + row) * a.q_ld + (size_t)h * (a.dim_p + a.rot_p);
-    if (gr * 8 < a.dim_p) return *reinterpret_cast<const frag*>(p + gr * 8);
-    const float* turn = a.turn + (size_t)(s.row0 + row) * a.rot_dims;
-    frag f;
-#pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      const int j = gr * 8 + e - a.dim_p;
-      f[e] = (T)(j < a.rot_dim ? turned([&](int i) { return (float)p[a.dim_p + i]; }, turn, a.rot_dims, j) : 0.f);
-    }
-    return f;
+    return *reinterpret_cast<const frag*>(reinterpret_cast<const T*>(a.q_t) + (size_t)(s.row0 + row) * a.q_ld + (size_t)h * (a.dim_p + a.rot_p) + gr * 8);
   }
   DEV frag k(int pos, int gr) const {
     const size_t r = key_row(pos);
@@ -155,7 +164,7 @@ struct LatentKeys {
   }
 };
 template <typename T, int KT, int VTL>
-__global__ __launch_bounds__(256) void latent_attn_kernel(const LatentArgs a) {
+ATTN_KERNEL(T) void latent_attn_kernel(const LatentArgs a) {
   const int h = blockIdx.y, tile = gridDim.x - 1 - blockIdx.x;  // (a sequence's last tiles have the most keys: they start first)
   const SeqDesc s = a.p.seqs[a.p.qtile[2 * tile]];
   if (s.len == 1) return;
@@ -357,30 +366,31 @@ int launch_latent_gather(hipStream_t st, const LatentArgs& a, bool f32) {
   else hipLaunchKernelGGL(latent_gather_kernel<bf16>, grid, dim3(256), 0, st, a);
   return DSK_OK;
 }
+int launch_latent_turn(hipStream_t st, const LatentArgs& a, bool f32) {
+  if (a.rot_dims < 2) return DSK_OK;
+  if (f32) hipLaunchKernelGGL(latent_turn_kernel<float>, dim3(a.p.rows), dim3(256), 0, st, a);
+  else hipLaunchKernelGGL(latent_turn_kernel<bf16>, dim3(a.p.rows), dim3(256), 0, st, a);
+  return DSK_OK;
+}
 int launch_latent_store(hipStream_t st, const LatentArgs& a, bool f32) {
   const dim3 grid(cdiv(a.p.rows, 4));
   if (f32) hipLaunchKernelGGL(latent_store_kernel<float>, grid, dim3(256), 0, st, a);
   else hipLaunchKernelGGL(latent_store_kernel<bf16>, grid, dim3(256), 0, st, a);
   return DSK_OK;
 }
-template <typename T, int KT, int VTL>
-static int attn_t(hipStream_t st, const LatentArgs& a) {
-  const size_t lds = attn_tile_lds<T>(a.dim_p + a.rot_p, a.vdim_p);
-  auto k = latent_attn_kernel<T, KT, VTL>;
-  HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
-  hipLaunchKernelGGL(k, dim3(a.p.n_qtiles, a.heads), dim3(256), lds, st, a);
-  return DSK_OK;
-}
 template <typename T>
-static int attn_dims(hipStream_t st, const LatentArgs& a) {
-  const int d = a.dim_p + a.rot_p;
-  if (d <= 128 && a.vdim_p <= 128) return attn_t<T, 4, 8>(st, a);
-  if (d <= 192 && a.vdim_p <= 128) return attn_t<T, 6, 8>(st, a);
-  return attn_t<T, 8, 16>(st, a);
+static int attn_t(hipStream_t st, const LatentArgs& a) {
+  return attn_sizes((a.dim_p + a.rot_p) >> 5, a.vdim_p >> 4, [&](auto kt, auto vt) -> int {
+    constexpr int KT = decltype(kt)::value, VTL = decltype(vt)::value, lds = attn_tile_lds<T, KT, VTL>();
+    auto k = latent_attn_kernel<T, KT, VTL>;
+    HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize, lds));
+    hipLaunchKernelGGL(k, dim3(a.p.n_qtiles, a.heads), dim3(256), lds, st, a);
+    return (int)DSK_OK;
+  }, "latent attention");
 }
 int launch_latent_attn(hipStream_t st, const LatentArgs& a, bool f32) {
   DSK_TRY(check_latent(a, f32));
-  return f32 ? attn_dims<float>(st, a) : attn_dims<bf16>(st, a);
+  return f32 ? attn_t<float>(st, a) : attn_t<bf16>(st, a);
 }
 template <typename T>
 static int few_t(hipStream_t st, const LatentArgs& a) {

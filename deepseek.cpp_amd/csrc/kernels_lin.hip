@@ -122,10 +122,6 @@ DEV const T* operand(const LinArgs& a, int feature) {
 // ---- prompts -------------------------------------------------------------------------------------
 // grid.x: row tiles of 128 (experts: entries of the tile table), grid.y: feature tiles of 128.
 // rows: a gather table (slot -> row) or nullptr; out rows are row0 + local row.
-// A block of activations (16 rows x 32 columns, bf16) arrives row by row, four lanes to the 64 bytes of a row; inside a row the groups of 8
-// columns are exchanged by the row's place so that the lanes that read one group of 16 rows meet every LDS bank once.
-DEV int block_group(int lane) { return (lane & 3) ^ (lane >> 4); }                                  // the group lane l of a load brings
-DEV int block_at(int lane) { return ((lane & 15) * 4 + ((lane >> 4) ^ ((lane >> 2) & 3))) * 16; }  // where lane l of an operand reads
 template <typename T>
 DEV void lin_body(const LinArgs& a, const int* gather, int row0, int n_rows, int f0, int k0, int k1, char* lds) {
   typedef typename Frag<T>::type frag;
@@ -142,7 +138,7 @@ DEV void lin_body(const LinArgs& a, const int* gather, int row0, int n_rows, int
     const int t = 2 * wave + i;
     const int rt = min(rt0 + t, a.rt - 1);  // (tiles past the end: any valid one, never stored)
     src_w[i] = reinterpret_cast<const char*>(a.w) + (size_t)rt * a.kt * 1024 + lane * 16;
-    int r = min(t * 16 + (sizeof(T) == 2 ? lane >> 2 : lane & 15), n_rows - 1);
+    int r = min(t * 16 + (sizeof(T) == 2 ? block_row(lane) : lane & 15), n_rows - 1);
     r = gather ? gather[row0 + r] : row0 + r;
     src_a[i] = operand<T>(a, f0) + (size_t)r * a.lda + (sizeof(T) == 2 ? block_group(lane) : lane >> 4) * 8;
   }
@@ -162,7 +158,7 @@ DEV void lin_body(const LinArgs& a, const int* gather, int row0, int n_rows, int
   auto read_a = [&](const char* buf, int slot) {
     frag f;
     if constexpr (sizeof(T) == 2) {
-      f = *reinterpret_cast<const frag*>(buf + 16 * 1024 + slot * AB + block_at(lane));
+      f = *reinterpret_cast<const frag*>(buf + 16 * 1024 + slot * AB + block_place(lane) * 16);
     } else {
       const f32x4 lo = *reinterpret_cast<const f32x4*>(buf + 16 * 1024 + slot * AB + lane * 16);
       const f32x4 hi = *reinterpret_cast<const f32x4*>(buf + 16 * 1024 + slot * AB + 1024 + lane * 16);
@@ -235,7 +231,7 @@ __global__ __launch_bounds__(512) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
   for (int i = 0; i < 2; ++i) {
     const int t = 2 * wave + i;
     src_w[i] = reinterpret_cast<const char*>(a.w) + ((size_t)min(rt0 + t, a.rt - 1) * a.kt + k0) * 1024 + lane * 16;
-    src_a[i] = reinterpret_cast<const char*>(operand<bf16>(a, f0) + (size_t)(row0 + min(t * 16 + (lane >> 2), n_rows - 1)) * a.lda + (size_t)k0 * 32 + block_group(lane) * 8);
+    src_a[i] = reinterpret_cast<const char*>(operand<bf16>(a, f0) + (size_t)(row0 + min(t * 16 + block_row(lane), n_rows - 1)) * a.lda + (size_t)k0 * 32 + block_group(lane) * 8);
   }
   auto stage = [&](int kt, char* buf) {  // (past the end: the last tile again, never read)
     kt = min(kt, n - 1);
@@ -256,7 +252,7 @@ __global__ __launch_bounds__(512) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
   };
   auto read = [&](const char* buf, Operands& o) {
 #pragma unroll
-    for (int j = 0; j < 4; ++j) o.x[j] = *reinterpret_cast<const bf16x8*>(buf + 16 * 1024 + (wn * 4 + j) * 1024 + block_at(lane));
+    for (int j = 0; j < 4; ++j) o.x[j] = *reinterpret_cast<const bf16x8*>(buf + 16 * 1024 + (wn * 4 + j) * 1024 + block_place(lane) * 16);
 #pragma unroll
     for (int i = 0; i < 8; ++i) o.w[i] = *reinterpret_cast<const bf16x8*>(buf + (wm * 8 + i) * 1024 + lane * 16);
   };

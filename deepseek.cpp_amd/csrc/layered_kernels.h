@@ -256,7 +256,7 @@ struct LatentArgs {
   void* cq_t;               // normed query latents [rows][cq_ld], zero up to a multiple of 64 columns
   int cq_ld;
   float* turn;              // cosines, then sines of a row's angles [rows][rot_dims]
-  const void* q_t;          // queries [rows][q_ld], per head [dim_p][rot_p], not rotated yet
+  void* q_t;                // queries [rows][q_ld], per head [dim_p][rot_p], not rotated yet
   int q_ld;
   void* lat_t;              // key workspace: latent rows [key rows][rank_p + rot_p]
   const void* kv_t;         // ... expanded [key rows][heads * dim_p + heads * vdim_p]
@@ -274,6 +274,7 @@ struct LatentArgs {
 int latent_keys(bool f32);
 int launch_latent_prep(hipStream_t st, const LatentArgs& a, bool f32);    // norms, rotation; single tokens' rows go into their rings
 int launch_latent_gather(hipStream_t st, const LatentArgs& a, bool f32);  // older rows from the rings into the key workspace
+int launch_latent_turn(hipStream_t st, const LatentArgs& a, bool f32);    // rotates the queries of portions of several tokens
 int launch_latent_attn(hipStream_t st, const LatentArgs& a, bool f32);    // portions of several tokens
 int launch_latent_store(hipStream_t st, const LatentArgs& a, bool f32);   // their rows into the rings
 int launch_latent_few(hipStream_t st, const LatentArgs& a, bool f32);     // single tokens: scores, weights, latent sums, values

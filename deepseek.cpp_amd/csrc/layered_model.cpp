@@ -981,6 +981,7 @@ int latent(LayeredModel* m, LatentArgs a, const LayerW& w, bool few) {
     DSK_TRY(launch_latent_gather(st, a, m->f32));
     const LinArgs ukv = to_t(lin(w.l_ukv, m->lat, w.rank_p + w.rot_p, a.p.key_rows), m->kv, a.kv_ld);
     DSK_TRY(run_lin(m, &ukv, 1, false));
+    DSK_TRY(launch_latent_turn(st, a, m->f32));
     DSK_TRY(launch_latent_attn(st, a, m->f32));
     DSK_TRY(launch_latent_store(st, a, m->f32));
   }

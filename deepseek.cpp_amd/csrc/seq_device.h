@@ -40,6 +40,13 @@ DEV f32x4 mma(const f32x8& w, const f32x8& a, f32x4 c) {
   return c;
 }
 
+// A block of 16 rows x 32 columns on its way from row-major memory to operands: loaded row by row, four lanes to a row, lane l's 8 columns
+// at place l of the block in LDS.  Inside a row the groups are exchanged by the row's place, so that the lanes that read one group of 16 rows
+// meet every LDS bank once.
+DEV int block_row(int lane) { return lane >> 2; }                                              // what lane l loads ...
+DEV int block_group(int lane) { return (lane & 3) ^ (lane >> 4); }
+DEV int block_place(int lane) { return (lane & 15) * 4 + ((lane >> 4) ^ ((lane >> 2) & 3)); }  // ... and the place that lane l of an operand reads
+
 template <typename T>
 DEV typename Frag<T>::four to_four(const f32x4& v) {
   return __builtin_convertvector(v, typename Frag<T>::four);

@@ -171,7 +171,7 @@ DEV void lin_body(const LinArgs& a, const int* gather, int row0, int n_rows, int
   for (int i = 0; i < 4; ++i)
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-  stage(k0, lds);
+  stage(k0, lds + ((k0 >> 1) & 1) * STAGE);
   for (int kt = k0; kt < k1; kt += 2) {
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this wave's loads into LDS; the barrier makes it everybody's
     __syncthreads();
@@ -433,8 +433,9 @@ static double lin_cost(int rows, int rt, int kt, int parts, bool big) {
   const int n = cdiv(rows, 128) * cdiv(rt, 8) * parts;
   return (n <= 256 ? 1.05 * k : cdiv(n, 512) * 1.3 * k) + 5 + sums;
 }
-static bool lin_big(int rows, int rt, int kt, int parts, int a_seg, bool f32) {
-  return !f32 && !(a_seg & 255) && lin_cost(rows, rt, kt, parts, true) < lin_cost(rows, rt, kt, parts, false);
+static bool lin_big(const LinArgs& a, int parts, bool f32) {
+  if (f32 || (a.a_seg & 255)) return false;
+  return a.tile ? a.tile == 256 : lin_cost(a.rows, a.rt, a.kt, parts, true) < lin_cost(a.rows, a.rt, a.kt, parts, false);
 }
 int lin_parts(int rows, int rt, int kt, bool f32, int most) {
   int best = 1;
@@ -455,7 +456,7 @@ int lin_parts_few(int rt, int kt, int most) {
 int launch_lin(hipStream_t st, const LinArgs& a, bool f32) {
   DSK_TRY(check_lin(a, "lin"));
   if ((a.a_seg & 127) || a.row_seq) DSK_FAIL(DSK_ERR_INVALID, "lin: %d features per operand", a.a_seg);
-  if (lin_big(a.rows, a.rt, a.kt, std::max(a.parts, 1), a.a_seg, f32)) {
+  if (lin_big(a, std::max(a.parts, 1), f32)) {
     const int row_tiles = cdiv(a.rows, 256), tiles = row_tiles * cdiv(a.rt, 16);
     DSK_TRY(allow_lds(lin_big_kernel, RING * 32 * 1024));
     hipLaunchKernelGGL(lin_big_kernel, dim3(tiles, std::max(a.parts, 1)), dim3(512), RING * 32 * 1024, st, a, row_tiles, tiles);

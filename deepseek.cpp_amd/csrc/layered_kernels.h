@@ -59,6 +59,7 @@ struct LinArgs {
   size_t a_stride;        // ... a_stride elements behind each other (launch_lin: a_seg is a multiple of 128, else of 16)
   int parts;              // > 1: k in `parts` ranges, each with a 32-bit output of its own (part_stride elements behind each other; n_wide = 0,
   size_t part_stride;     // LIN_STORE); the reader adds them up
+  int tile;               // launch_lin: 0 chooses, 128 or 256 (bf16)
   const int* row_seq;     // launch_lin_few: output row i reads the first row of sequence row_seq[i] of seqs (nullptr: row i)
   const SeqDesc* seqs;
 };

@@ -124,6 +124,7 @@ struct LayeredModel : ModelHead {
   DescBuf big, small;
   int last_rows = 0;
   bool chunk_scan = true;
+  int tile = 0;                     // of prompt products (LinArgs::tile)
   ChunkScan scan{};                 // operands of the recurrences over chunks (kernels_chunk_scan.hip)
   int max_chunks = 0;
   float* attn_part = nullptr;       // parts of attention outputs (kernels_mix_few.hip)
@@ -683,7 +684,11 @@ LinArgs mix_lin(LayeredModel* m, const PackedMat& w, const void* a, int lda, int
 }
 int run_lin(LayeredModel* m, const LinArgs* a, int n, bool few) {
   if (few) return launch_lin_few(m->ctx->stream, a, n, m->f32);
-  for (int i = 0; i < n; ++i) DSK_TRY(launch_lin(m->ctx->stream, a[i], m->f32));
+  for (int i = 0; i < n; ++i) {
+    LinArgs l = a[i];
+    l.tile = m->tile;
+    DSK_TRY(launch_lin(m->ctx->stream, l, m->f32));
+  }
   return DSK_OK;
 }
 
@@ -1582,6 +1587,10 @@ int set_options(LayeredModel* m, const char* options) {
     } else if (k == "decode_graph") m->use_graph = v != 0;
     else if (k == "fused_decode") m->fused_decode = v != 0;
     else if (k == "chunk_scan") m->chunk_scan = v != 0;
+    else if (k == "prompt_tile") {
+      if (v != 0 && v != 128 && v != 256) DSK_FAIL(DSK_ERR_INVALID, "open: prompt_tile %d (0, 128, 256)", v);
+      m->tile = v;
+    }
     else DSK_FAIL(DSK_ERR_INVALID, "open: unknown option '%s'", k.c_str());
     p = e ? e + 1 : nullptr;
   }

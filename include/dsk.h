@@ -450,7 +450,8 @@ int dsk_bench_router(dsk_ctx* ctx, int n_routed, int dim, int ksplit, int flags,
  * DSK_DTYPE_BF16 = matrix products and activations in bfloat16 with 32-bit accumulation, DSK_DTYPE_F32 = everything in 32-bit.
  * options: "key=value[,key=value]" or NULL.  Layered models: "piece_tokens" (tokens one pass of a step runs, default 2048),
  * "decode_graph" (1: steps of single tokens replay a captured graph), "fused_decode" (1: the fused launches for such steps),
- * "chunk_scan" (1: prompts run their recurrences over chunks of tokens as matrix products; 0: token by token). */
+ * "chunk_scan" (1: prompts run their recurrences over chunks of tokens as matrix products; 0: token by token), "prompt_tile"
+ * (tiles of prompt products in bfloat16: 128 or 256 rows and features; 0, the default: whichever is faster). */
 enum { DSK_DTYPE_BF16 = 0, DSK_DTYPE_F32 = 1 };
 int dsk_dir_architecture(const char* dir, char* out, int cap); /* needs no GPU */
 int dsk_config_check(const char* config_json);                  /* is this the configuration of a layered design? needs no GPU */

@@ -156,6 +156,23 @@ def test_feed_forward(case, p, q):
     case(alone(dict(U.wkv(1, 8), mlp=U.dense(300))), edit=edit).check_trace(140, cuts=([139], list(range(130, 140))))
 
 
+@pytest.mark.parametrize("ff", [576, 1152, 1184, 2112, 4100])
+def test_products_split_over_k(case, ff):
+    """down products (and a mixer's output product) long enough to be split into parts, of an odd and an even number of steps"""
+    K = case(U.sandwich([dict(U.head_delta(9, 3, 8, 128, 4), mlp=U.dense(ff)), dict(U.wkv(2, 36), mlp=U.dense(ff))], width=88))
+    K.check_trace(150, tol=TOL, cuts=([20], list(range(130, 150))))
+
+
+@pytest.mark.parametrize("rows", [17, 300, 600])
+def test_prompt_tiles_of_both_sizes(case, rows):
+    c = U.sandwich([dict(U.wkv(4, 64), mlp=U.dense(1152)), dict(U.head_delta(5, 5, 64, 64, 4), mlp=U.dense(700)), U.latent(6, 64, 32, 48, 90, 130, 100, 0.1)], width=330)
+    runs = [case(c, dtype="bfloat16", options=f"prompt_tile={tile}") for tile in (128, 256)]
+    t = runs[0].tokens(rows)
+    want = runs[0].want(t)
+    a, b = (K.got(t) for K in runs)
+    assert U.err(a, want) < U.B16 and U.err(b, want) < U.B16 and U.err(a, b) < U.B16
+
+
 def test_layers_without_a_feed_forward_in_any_order(case):
     K = case(U.sandwich([U.no_ff(U.head_delta()), U.no_ff(U.latent()), U.wkv(), U.no_ff(U.wkv(1, 24)), U.latent(2, 16, 8, 16, 12, 20, 6)]))
     K.check_trace(60, tol=TOL, cuts=([9], list(range(50, 60))))
